@@ -42,6 +42,7 @@ from .. import ops
 from ..engine.state_pool import StatePool
 from ..parallel.dist import DistContext, get_context
 from .common import ForwardBatch
+from .hybrid_base import HybridDecoderBase
 
 MIXERS = ("parallel", "mamba2")
 RGLRU_C = 8.0    # log a = -RGLRU_C * r * softplus(lam)
@@ -201,11 +202,8 @@ def random_state(cfg: RonavikConfig, seed: int = 0) -> Dict[str, torch.Tensor]:
     return sd
 
 
-class RonavikModel:
+class RonavikModel(HybridDecoderBase):
     """Weights (plain tensors) + forward for the serving engine (the hooks of LlamaModel / PinavikModel)."""
-
-    has_recurrent_state = True       # no prefix-cache reuse: a cached prefix has no recurrent state to resume from
-    attention_backend = "window"     # the paged window / sigmoid attention kernels: no flash-attention tile lists
 
     def __init__(self, cfg: RonavikConfig, device=None, dtype=torch.bfloat16, dist_ctx: DistContext | None = None,
                  state_slots: Optional[int] = None):
@@ -226,7 +224,6 @@ class RonavikModel:
         self.pool = StatePool(state_slots or int(os.environ.get("GAI_LINEAR_STATE_SLOTS", "64")), self.device)
         self.state: Dict[int, Dict[str, torch.Tensor]] = {}
         self.capture_residuals: Optional[list] = None  # numerics debugging: the residual stream after every layer
-        self._i32 = dict(dtype=torch.int32, device=self.device)
 
     # ------------------------------------------------------------------ engine sizing hooks
     def kv_layout(self) -> List[Tuple[int, int, int]]:
@@ -289,22 +286,8 @@ class RonavikModel:
         self._alloc_state()
         return self
 
-    load_hf_state = load_state
-
-    def load_safetensors_dir(self, path: str):
-        from safetensors.torch import load_file
-
-        sd = {}
-        for f in sorted(os.listdir(path)):
-            if f.endswith(".safetensors"):
-                sd.update(load_file(os.path.join(path, f)))
-        return self.load_state(sd)
-
     def random_init(self, seed: int = 0):
         return self.load_state(random_state(self.cfg, seed))
-
-    def num_params(self) -> int:
-        return sum(t.numel() for t in self.w.values())
 
     # ------------------------------------------------------------------ recurrent state slots
     def _alloc_state(self):
@@ -320,49 +303,6 @@ class RonavikModel:
                 C = m["heads"] * m["vdim"] + 2 * m["groups"] * m["state"]
                 self.state[i] = dict(conv=self.pool.add(tag + "conv", (m["conv"] - 1, C)),
                                      S=self.pool.add(tag + "S", (m["heads"], m["state"], m["vdim"])))
-
-    def set_state_slots(self, n: int):
-        """Engine hook: size the state pool for n live sequences (before any request is admitted)."""
-        if n != self.pool.n_slots:
-            self.pool = StatePool(n, self.device)
-            if self.w:
-                self._alloc_state()
-
-    def release_request(self, sid: int):
-        self.pool.release(sid)
-
-    def prepare_batch(self, fb: ForwardBatch):
-        """Engine hook: one (cu, slot, ctx, page table) row per sequence of the step - prompt portions first, then
-        single decoded tokens - and fresh state for sequences that start at position 0."""
-        P = len(fb.prefill_qlen)
-        nd = fb.num_tokens - fb.num_prefill_tokens
-        pctx = fb.prefill_ctx_host or []
-        dctx = fb.decode_ctx_host or []
-        sids = fb.seq_ids or []
-        slots = [self.pool.slot(sid, pctx[i] == fb.prefill_qlen[i]) for i, sid in enumerate(sids[:P])]
-        slots += [self.pool.slot(sid, dctx[j] == 1 if j < len(dctx) else False) for j, sid in enumerate(sids[P:])]
-        cu = [0]
-        for n in fb.prefill_qlen:
-            cu.append(cu[-1] + n)
-        cu += [cu[-1] + j + 1 for j in range(nd)]
-        dev = self.device
-        extra = dict(cu=torch.tensor(cu, dtype=torch.int32).to(dev, non_blocking=True),
-                     slots=torch.tensor(slots, dtype=torch.int32).to(dev, non_blocking=True))
-        parts_c = [t for t in (fb.prefill_ctx if P else None, fb.decode_ctx if nd else None) if t is not None]
-        parts_b = [t for t in (fb.prefill_block_tables if P else None, fb.decode_block_tables if nd else None)
-                   if t is not None]
-        extra["ctx"] = parts_c[0] if len(parts_c) == 1 else torch.cat(parts_c)
-        extra["bt"] = parts_b[0] if len(parts_b) == 1 else torch.cat(parts_b)
-        fb.extra = extra
-
-    def graph_static_inputs(self, bs: int) -> dict:
-        """Static inputs of a captured decode graph of bs rows (the engine's ctx / page-table tensors complete them)."""
-        return dict(cu=torch.arange(bs + 1, **self._i32), slots=torch.full((bs,), self.pool.pad_slot, **self._i32))
-
-    def fill_graph_inputs(self, extra: dict, seq_ids, n: int):
-        ids = torch.tensor([self.pool.slot(s, False) for s in seq_ids] +
-                           [self.pool.pad_slot] * (extra["slots"].numel() - n), dtype=torch.int32)
-        extra["slots"].copy_(ids, non_blocking=True)
 
     # ------------------------------------------------------------------ mixers
     def _parallel(self, h, i, fb, kv, seq):
