@@ -13,6 +13,7 @@ from .clip import ClipConfig, ClipModel
 from .decoder_reranker import DecoderRerankerConfig, DecoderRerankerModel
 from .lituvik import LituvikConfig, LituvikModel
 from .llama import LlamaConfig, LlamaModel
+from .luketar import LuketarConfig, LuketarModel
 from .mixtral import MixtralConfig, MixtralModel
 from .mllama import MllamaConfig, MllamaModel
 from .opt import OPTConfig, OPTModel
@@ -53,6 +54,10 @@ LLM_PRESETS = {
     # sigmoid routing over clamped gated experts, per-layer token input)
     "tiny-vipolix": ("tiny-vipolix", lambda: VipolixConfig.tiny()),
     "vipolix-1b": ("vipolix-1b", lambda: VipolixConfig.sized(2048, 12, 5632, 16, 128)),
+    # hybrid of latent attention with sinks and matrix-memory LSTM layers (residual streams joined by hyper-connections,
+    # routed clamped gated experts plus a shared expert)
+    "tiny-luketar": ("tiny-luketar", lambda: LuketarConfig.tiny()),
+    "luketar-1b": ("luketar-1b", lambda: LuketarConfig.sized(2048, 12, 5632, 16, 128)),
     "opt-125m": ("facebook/opt-125m", lambda: OPTConfig.opt_125m()),
     "mixtral-8x7b": ("mistralai/mixtral-8x7b-instruct-v0.1", lambda: MixtralConfig.mixtral_8x7b()),
     "tiny-moe": ("tiny-moe", lambda: MixtralConfig.tiny_moe()),
@@ -98,6 +103,8 @@ def build_llm(preset: str = "llama3-8b", weights: Optional[str] = None, device=N
             m = LituvikModel(LituvikConfig.from_json(weights), device=device, dtype=dtype or torch.bfloat16)
         elif arch == "vipolix":
             m = VipolixModel(VipolixConfig.from_json(weights), device=device, dtype=dtype or torch.bfloat16)
+        elif arch == "luketar":
+            m = LuketarModel(LuketarConfig.from_json(weights), device=device, dtype=dtype or torch.bfloat16)
         elif arch == "opt":
             m = OPTModel(OPTConfig.from_hf(weights), device=device)
         elif arch == "mixtral":
@@ -140,6 +147,9 @@ def build_llm(preset: str = "llama3-8b", weights: Optional[str] = None, device=N
         vocab = cfg.vocab_size
     elif isinstance(cfg, VipolixConfig):
         m = VipolixModel(cfg, device=device, dtype=dtype or torch.bfloat16).random_init(seed)
+        vocab = cfg.vocab_size
+    elif isinstance(cfg, LuketarConfig):
+        m = LuketarModel(cfg, device=device, dtype=dtype or torch.bfloat16).random_init(seed)
         vocab = cfg.vocab_size
     else:
         m = LlamaModel(cfg, device=device).random_init(seed)

@@ -834,9 +834,17 @@ def moe_route(logits: torch.Tensor, k: int, renorm: bool = True, score: str = "s
     eps is added to the sum that renormalises them. Sigmoid scoring with bias, groups or scale: the choice is made on
     sigmoid score + bias; groups = (count, keep) cuts the expert list into `count` contiguous parts of equal size, ranks
     each by its two best choice scores added up and confines the choice to the `keep` best parts; the
-    weights are the chosen plain scores over their sum (+ eps), times scale."""
-    if score not in ("softmax", "sigmoid"):
+    weights are the chosen plain scores over their sum (+ eps), times scale. score "chosen": bias is part of the logits;
+    the choice is made on logits + bias and the weights are the softmax over the chosen ones only."""
+    if score not in ("softmax", "sigmoid", "chosen"):
         raise ValueError(f"moe_route: unknown score function {score!r}")
+    if score == "chosen":
+        if not logits.is_cuda:
+            return ref.moe_route_chosen(logits, k, bias)
+        ids = torch.empty(logits.shape[0], k, dtype=torch.int32, device=logits.device)
+        w = torch.empty(logits.shape[0], k, dtype=torch.float32, device=logits.device)
+        native().moe_route_chosen(logits, k, ids, w, bias)
+        return ids, w
     if score == "sigmoid" and (bias is not None or groups is not None or scale != 1.0 or eps):
         ng, keep = (int(groups[0]), int(groups[1])) if groups is not None else (1, 1)
         E = logits.shape[1]
@@ -1177,12 +1185,12 @@ def qknorm_kv_write(q, k, v, wq, wk, slots, k_cache, v_cache, H: int, G: int, DK
 
 def window_attention(q, k_cache, v_cache, block_tables, cu_q, ctx, H: int, G: int, DK: int, DV: int, scale: float,
                      softcap: float = 0.0, window: int = 0, r1=None, r2=None, gate=None, chunk: int = 0, head_scale=None,
-                     sink: Optional[float] = None, out=None, out_scale: float = 1.0):
+                     sink=None, out=None, out_scale: float = 1.0):
     """Paged softmax attention over the visible keys j <= i: the last `window` ones (window > 0), those of the query's
     own chunk of positions, floor(j / chunk) == floor(i / chunk) (chunk > 0), or all. Scores are capped by softcap *
     tanh(s / softcap) and lowered by r1_h ln(1 + r2_h distance); head_scale (fp32 [H]) multiplies the scores of a head;
-    sink (a score) adds exp(sink) to the softmax denominator without a value (sink = 0: one is added). Output
-    [T, H * DV] times out_scale, times sigmoid(gate) when given (`out` may be a column slice of a wider buffer)."""
+    sink (a score, or an fp32 [H] tensor of scores, one per head) adds exp(sink) to the softmax denominator without a
+    value (sink = 0: one is added). Output [T, H * DV] times out_scale, times sigmoid(gate) when given (`out` may be a column slice of a wider buffer)."""
     if not q.is_cuda:
         if chunk or head_scale is not None or sink is not None or out_scale != 1.0:
             if softcap or r1 is not None or gate is not None:
@@ -1197,9 +1205,10 @@ def window_attention(q, k_cache, v_cache, block_tables, cu_q, ctx, H: int, G: in
     T, S = q.shape[0], ctx.numel()
     ns = native().sigmoid_attention_splits(T, S, H)
     part = torch.empty(ns * T * H * (DV + 2), dtype=torch.float32, device=q.device) if ns > 1 else None
+    hs = sink if isinstance(sink, torch.Tensor) else None
     native().window_attention(q, k_cache, v_cache, block_tables, cu_q, ctx, out, H, G, DK, DV, float(scale),
                               float(softcap or 0.0), int(window or 0), r1, r2, gate, None, False, float(out_scale), part,
-                              int(chunk or 0), head_scale, None if sink is None else float(sink))
+                              int(chunk or 0), head_scale, None if sink is None or hs is not None else float(sink), hs)
     return out
 
 
@@ -1482,3 +1491,63 @@ def dplr_scan(q, k, v, decay, av, bv, state, cu, slots, q_scale: float = 1.0):
     ws = torch.empty(nws, dtype=torch.float32, device=q.device) if nws else None
     native().dplr_scan(q, k, v, decay, av, bv, state, cu, slots, out, float(q_scale), ws)
     return out
+
+
+# ---------------------------------------------------------------------------------------------
+# parallel residual streams, latent attention with a query latent, matrix-memory LSTM
+# ---------------------------------------------------------------------------------------------
+def hyper_connect(X, x0=None, y=None, mix=None, out_w=None, in_w=None, norm_w=None, eps: float = 1e-6, out_dtype=None):
+    """Residual streams X (fp32 [T, s, D], in place) of a hyper-connected decoder, one pass between two sublayers: close
+    the sublayer that produced y - X_t <- sum_s mix[s, t] X_s + out_w[t] * y, all streams from the old ones - and open the
+    next one: u = sum_s in_w[s] X_s, layer norm (norm_w, no bias) of u in out_dtype. y None: only open; in_w None: only
+    close. x0 (fp32 [T, D]): the old streams are all equal to x0 (the embedding output) and X is only written."""
+    if not X.is_cuda:
+        return ref.hyper_connect(X, x0, y, mix, out_w, in_w, norm_w, eps, out_dtype)
+    out = torch.empty(X.shape[0], X.shape[2], dtype=out_dtype, device=X.device) if in_w is not None else None
+    native().hyper_connect(X, x0, y, mix, out_w, in_w, norm_w, float(eps), out)
+    return out
+
+
+def latent_norm_write(dq, wq, dkv, wkv, slots, k_cache, v_cache, eps: float):
+    """Latent attention whose queries go through a latent too and which rotates nothing: returns rmsnorm(dq) * wq and
+    writes the key / value latent rmsnorm(dkv) * wkv as the token's whole cache row (K page row and V^T page of one kv
+    head). dq / dkv may be column slices of one projection; both norms in one launch, fp32 statistics."""
+    if not dq.is_cuda:
+        return ref.latent_norm_write(dq, wq, dkv, wkv, slots, k_cache, v_cache, eps)
+    out = torch.empty(dq.shape, dtype=dq.dtype, device=dq.device)
+    native().latent_norm_write(dq, wq, dkv, wkv, slots, out, k_cache, v_cache, float(eps))
+    return out
+
+
+def head_linear(x, W, gate=None):
+    """Per-head products y[t, h, :] = W[h] x[t, h, :] for x [T, H * K], W [H, N, K] -> [T, H * N], times sigmoid(gate)
+    ([T, H * N], may be a column slice) when given: the folds of latent attention (queries through the key expansion,
+    weighted latents through the value expansion with the output gate) without transposed copies."""
+    if not x.is_cuda:
+        return ref.head_linear(x, W, gate)
+    H, N, K = W.shape
+    out = torch.empty(x.shape[0], H * N, dtype=x.dtype, device=x.device)
+    native().head_linear(x, W, gate, out)
+    return out
+
+
+def mlstm(q, k, v, ig, fg, ib, fb, cap: float, gate, norm_w, S, n, m, cu, slots, q_scale: float, eps: float,
+          den_eps: float, out_dtype):
+    """Matrix-memory LSTM (mLSTM) mixer core, gates and norms included. Per head, log input gate i = cap *
+    tanh((ig + ib) / cap) and log forget gate f = logsigmoid(cap * tanh((fg + fb) / cap)); a running maximum m keeps the
+    exponentials bounded: m_t = max(f + m_(t-1), i), S_t = e^(f + m_(t-1) - m_t) S_(t-1) + e^(i - m_t) k v^T, n_t likewise
+    with k alone, o = S_t^T (q_scale q) / (max(|n_t . q_scale q|, e^(-m_t)) + den_eps); then a per-head RMS norm (eps),
+    times norm_w [H * DV], times sigmoid(gate). q / k [T, H * DK], v / gate [T, H * DV] in the activation dtype and
+    ig / fg fp32 [T, H] (column slices of projections); states S [slots, H, DK, DV], n [slots, H, DK], m [slots, H] fp32 in
+    place. Steps of single tokens run one fused kernel per (sequence, head); portions run the chunk form on the fp32
+    matrix cores."""
+    if not q.is_cuda:
+        return ref.mlstm(q, k, v, ig, fg, ib, fb, cap, gate, norm_w, S, n, m, cu, slots, q_scale, eps, den_eps, out_dtype)
+    H, DK, DV = S.shape[1:]
+    T, nseq = q.shape[0], slots.numel()
+    y = torch.empty(T, H * DV, dtype=out_dtype, device=q.device)
+    nws = native().mlstm_ws_floats(T, nseq, H, DK, DV)
+    ws = torch.empty(nws, dtype=torch.float32, device=q.device) if nws else None
+    native().mlstm(q, k, v, ig, fg, ib, fb, float(cap), gate, norm_w, S, n, m, cu, slots, float(q_scale), float(eps),
+                   float(den_eps), y, ws)
+    return y

@@ -928,7 +928,7 @@ def masked_attention(q, k_cache, v_cache, block_tables, cu_q, ctx, H, G, DK, DV,
                      out_scale):
     """Softmax attention over the visible keys j <= i: the last `window` ones (window > 0), those of the query's own
     chunk of positions floor(i / chunk) = floor(j / chunk) (chunk > 0), or all. head_scale [H] multiplies the scores of
-    a head; sink (a score, or None) adds exp(sink) to the softmax denominator without adding a value."""
+    a head; sink (a score, fp32 [H] scores, or None) adds exp(sink) to the softmax denominator without adding a value."""
     T = q.numel() // (H * DK)
     q3 = q.float().view(T, H, DK)
     out = torch.zeros(T, H, DV)
@@ -953,12 +953,13 @@ def masked_attention(q, k_cache, v_cache, block_tables, cu_q, ctx, H, G, DK, DV,
             sc = (q3[b:e, h] @ K[h // (H // G)].t()) * (scale * (float(head_scale[h]) if head_scale is not None else 1.0))
             sc = sc.masked_fill(~vis, float("-inf"))
             m = sc.max(-1, keepdim=True).values
-            if sink is not None:
-                m = m.clamp(min=float(sink))
+            sk = float(sink[h]) if isinstance(sink, torch.Tensor) else sink
+            if sk is not None:
+                m = m.clamp(min=float(sk))
             p = torch.exp(sc - m)
             den = p.sum(-1, keepdim=True)
-            if sink is not None:
-                den = den + torch.exp(float(sink) - m)
+            if sk is not None:
+                den = den + torch.exp(float(sk) - m)
             out[b:e, h] = (p / den) @ V[h // (H // G)]
     return (out.reshape(T, H * DV) * float(out_scale)).to(q.dtype)
 
@@ -1041,3 +1042,78 @@ def moe_gemm_clamp_glu(A, a_rows, W, offs, rows_total, limit):
             y = (rows.float() @ W[e].float().t()).view(rows.shape[0], N // 32, 2, 16)
             C[o[e]:o[e + 1]] = clamp_glu(y[:, :, 0], y[:, :, 1], limit).reshape(rows.shape[0], N // 2).to(A.dtype)
     return C
+
+
+# ---------------------------------------------------------------------------------------------
+# parallel residual streams (hyper-connections) around layer-normed sublayers, latent attention with a query latent and
+# learned sinks, matrix-memory LSTM, routing by softmax over the chosen logits
+# ---------------------------------------------------------------------------------------------
+def hyper_connect(X, x0, y, mix, out_w, in_w, norm_w, eps, out_dtype):
+    """X fp32 [T, s, D] in place. x0 given: every old stream is x0 [T, D]. y given: X_t <- sum_s mix[s, t] X_s + out_w[t] y.
+    in_w given: u = sum_s in_w[s] X_s, returned layer-normed (weight norm_w, no bias) in out_dtype."""
+    old = x0.float()[:, None, :].expand_as(X) if x0 is not None else X
+    new = old
+    if y is not None:
+        new = torch.einsum("bsd,st->btd", old, mix.float()) + out_w.float()[None, :, None] * y.float()[:, None, :]
+    if new is not X:
+        X.copy_(new.clone())
+    if in_w is None:
+        return None
+    u = torch.einsum("bsd,s->bd", X, in_w.float())
+    d = u - u.mean(-1, keepdim=True)
+    return (d * torch.rsqrt(d.pow(2).mean(-1, keepdim=True) + eps) * norm_w.float()).to(out_dtype)
+
+
+def latent_norm_write(dq, wq, dkv, wkv, slots, k_cache, v_cache, eps):
+    """Both latents of latent attention without rotation: c = rmsnorm(dkv) * wkv is the cache row (K page row and V^T page
+    of one kv head); returns rmsnorm(dq) * wq."""
+    T = dq.shape[0]
+    n = lambda t, w: t.float() * torch.rsqrt(t.float().pow(2).mean(-1, keepdim=True) + eps) * w.float()  # noqa: E731
+    c = n(dkv, wkv).to(k_cache.dtype)
+    s = slots[:T].long()
+    k_cache[s // BLOCK, 0, s % BLOCK] = c
+    v_cache[s // BLOCK, 0, :, s % BLOCK] = c
+    return n(dq, wq).to(dq.dtype)
+
+
+def head_linear(x, W, gate):
+    """Per-head products y[t, h] = W[h] x[t, h] (W [H, N, K], x [T, H * K]), times sigmoid(gate) element by element."""
+    H, N, K = W.shape
+    y = torch.einsum("thk,hnk->thn", x.float().reshape(-1, H, K), W.float()).reshape(-1, H * N)
+    if gate is not None:
+        y = y * torch.sigmoid(gate.float())
+    return y.to(x.dtype)
+
+
+def mlstm(q, k, v, ig, fg, ib, fb, cap, gate, norm_w, S, n, m, cu, slots, q_scale, eps, den_eps, out_dtype):
+    """Matrix-memory LSTM. Log gates i = cap tanh((ig + ib) / cap), f = logsigmoid(cap tanh((fg + fb) / cap));
+    m_t = max(f + m, i); S_t = e^(f + m - m_t) S + e^(i - m_t) k v^T, n_t likewise with k alone;
+    o = S_t^T q / (max(|n_t . q|, e^(-m_t)) + den_eps); per-head RMS norm, times norm_w, times sigmoid(gate)."""
+    H, DK, DV = S.shape[1:]
+    T = q.shape[0]
+    q3 = q.float().reshape(T, H, DK) * float(q_scale)
+    k3, v3 = k.float().reshape(T, H, DK), v.float().reshape(T, H, DV)
+    soft = lambda z, b: float(cap) * torch.tanh((z.float() + b.float()) / float(cap))  # noqa: E731
+    i_, f_ = soft(ig, ib), F.logsigmoid(soft(fg, fb))
+    out = torch.empty(T, H, DV)
+    for lo, hi, s in _seqs(cu, slots):
+        A, nn, mm = S[s], n[s], m[s]
+        for t in range(lo, hi):
+            m2 = torch.maximum(f_[t] + mm, i_[t])
+            a, b = torch.exp(f_[t] + mm - m2), torch.exp(i_[t] - m2)
+            A = a[:, None, None] * A + (b[:, None] * k3[t])[:, :, None] * v3[t][:, None, :]
+            nn = a[:, None] * nn + b[:, None] * k3[t]
+            mm = m2
+            den = torch.maximum((nn * q3[t]).sum(-1).abs(), torch.exp(-mm)) + den_eps
+            out[t] = torch.einsum("hkv,hk->hv", A, q3[t]) / den[:, None]
+        if hi > lo:
+            S[s], n[s], m[s] = A, nn, mm
+    y = out * torch.rsqrt(out.pow(2).mean(-1, keepdim=True) + eps)
+    return (y.reshape(T, H * DV) * norm_w.float() * torch.sigmoid(gate.float())).to(out_dtype)
+
+
+def moe_route_chosen(logits, k, bias):
+    """The k experts with the largest logits + bias; weights = softmax over those logits only."""
+    z = logits.float() + bias.float() if bias is not None else logits.float()
+    v, ids = torch.topk(z, k, dim=-1)
+    return ids.int(), torch.softmax(v, -1)
