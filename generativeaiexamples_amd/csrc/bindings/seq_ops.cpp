@@ -1,5 +1,5 @@
 // PyTorch bindings of the sequence-mixer kernels with a 32-bit residual / state (norm_f32.hip, attention_window.hip,
-// recurrent.hip). Shape / dtype checks on the host, a launch on the current stream, no allocation: graph-capturable.
+// recurrent.hip, hyper.hip, head_linear.hip, mlstm.hip). Shape / dtype checks on the host, a launch on the current stream, no allocation: graph-capturable.
 // Activation tensors are bf16 or fp32 (all of one call alike); per-channel tables and states are fp32.
 #include <torch/extension.h>
 #include <c10/hip/HIPStream.h>
@@ -182,7 +182,8 @@ void window_attention(const Tensor& q, const Tensor& k_cache, const Tensor& v_ca
                       double scale, double softcap, int64_t window, const optional<Tensor>& r1,
                       const optional<Tensor>& r2, const optional<Tensor>& gate, const optional<Tensor>& sig_bias,
                       bool sigmoid, double out_scale, const optional<Tensor>& part, int64_t chunk,
-                      const optional<Tensor>& head_scale, const optional<double>& sink) {
+                      const optional<Tensor>& head_scale, const optional<double>& sink,
+                      const optional<Tensor>& head_sink) {
   const int dt = act_dt(q, "q");
   same_dt(out, dt, "out");
   check_cache(k_cache, v_cache, dt, G, DK, DV);
@@ -194,6 +195,7 @@ void window_attention(const Tensor& q, const Tensor& k_cache, const Tensor& v_ca
                   block_tables.size(0) >= S, "window_attention: out / cu_q / block table shapes");
   if (sig_bias) TORCH_CHECK(sigmoid && sig_bias->numel() == H, "window_attention: one sigmoid bias per head");
   if (head_scale) TORCH_CHECK(!sigmoid && head_scale->numel() == H, "window_attention: one score scale per head, softmax mode");
+  if (head_sink) TORCH_CHECK(!sigmoid && !sink && head_sink->numel() == H, "window_attention: one sink score per head, softmax mode");
   TORCH_CHECK(chunk >= 0 && (!sigmoid || (chunk == 0 && !sink)), "window_attention: chunks and sinks go with the softmax mode");
   if (sigmoid) TORCH_CHECK(!gate && !r1 && softcap == 0.0, "window_attention: sigmoid mode takes no cap, distance term or gate");
   TORCH_CHECK(r1.has_value() == r2.has_value(), "window_attention: r1 and r2 come together");
@@ -217,7 +219,7 @@ void window_attention(const Tensor& q, const Tensor& k_cache, const Tensor& v_ca
                        r2 ? f32(*r2, "r2") : nullptr, gate ? gate->data_ptr() : nullptr, ldg,
                        sig_bias ? f32(*sig_bias, "sig_bias") : nullptr, sigmoid ? 1 : 0, (float)out_scale, dt,
                        cur_stream(), partp, (int)chunk, head_scale ? f32(*head_scale, "head_scale") : nullptr, sink ? 1 : 0,
-                       sink ? (float)*sink : 0.f);
+                       sink ? (float)*sink : 0.f, head_sink ? f32(*head_sink, "head_sink") : nullptr);
 }
 
 void rotary_kv_write(const Tensor& q, const Tensor& k, const Tensor& v, const Tensor& positions, const Tensor& slots,
@@ -555,10 +557,107 @@ void selective_scan(const Tensor& x, const Tensor& dt, const Tensor& dt_bias, co
                      I, N, dtt, cur_stream());
 }
 
+void latent_norm_write(const Tensor& dq, const Tensor& wq, const Tensor& dkv, const Tensor& wkv, const Tensor& slots,
+                       Tensor& q_out, Tensor& k_cache, Tensor& v_cache, double eps) {
+  const int dt = act_dt(dq, "dq");
+  same_dt(dkv, dt, "dkv");
+  same_dt(q_out, dt, "q_out");
+  const int ldq = row_stride(dq, "dq"), ldk = row_stride(dkv, "dkv");
+  const int T = dq.size(0), RQ = dq.size(1), R = dkv.size(1);
+  check_cache(k_cache, v_cache, dt, 1, R, R);
+  TORCH_CHECK(dkv.size(0) == T && wq.numel() == RQ && wkv.numel() == R && slots.numel() >= T && q_out.is_contiguous() &&
+                  q_out.numel() == dq.numel(), "latent_norm_write: shapes");
+  gai_latent_norm_write(dq.data_ptr(), ldq, f32(wq, "wq"), dkv.data_ptr(), ldk, f32(wkv, "wkv"), i32(slots, "slots"),
+                        q_out.data_ptr(), k_cache.data_ptr(), v_cache.data_ptr(), T, RQ, R, (float)eps, dt, cur_stream());
+}
+
+void hyper_connect(Tensor& X, const optional<Tensor>& x0, const optional<Tensor>& y, const optional<Tensor>& mix,
+                   const optional<Tensor>& out_w, const optional<Tensor>& in_w, const optional<Tensor>& norm_w, double eps,
+                   const optional<Tensor>& out) {
+  TORCH_CHECK(X.dim() == 3, "hyper_connect: X [T, streams, D]");
+  const int T = X.size(0), ns = X.size(1), D = X.size(2);
+  if (x0) TORCH_CHECK(x0->numel() == (int64_t)T * D, "hyper_connect: x0 [T, D]");
+  int dy = 0, od = 0, ldy = 0;
+  if (out) {
+    od = dy = act_dt(*out, "out");
+    TORCH_CHECK(out->is_contiguous() && out->numel() == (int64_t)T * D, "hyper_connect: out [T, D]");
+  }
+  if (y) {
+    dy = act_dt(*y, "y");
+    ldy = row_stride(*y, "y");
+    TORCH_CHECK(y->size(0) == T && y->size(1) == D && mix && mix->numel() == ns * ns && out_w && out_w->numel() == ns,
+                "hyper_connect: y [T, D] with mix [streams, streams] and out weights [streams]");
+  }
+  TORCH_CHECK(in_w.has_value() == out.has_value() && norm_w.has_value() == out.has_value() && (y || out || x0),
+              "hyper_connect: input weights, norm weight and output come together; something to do");
+  if (in_w) TORCH_CHECK(in_w->numel() == ns && norm_w->numel() == D, "hyper_connect: in weights [streams], norm weight [D]");
+  gai_hyper_connect(f32w(X, "X"), x0 ? f32(*x0, "x0") : nullptr, y ? y->data_ptr() : nullptr, ldy,
+                    y ? f32(*mix, "mix") : nullptr, y ? f32(*out_w, "out_w") : nullptr, in_w ? f32(*in_w, "in_w") : nullptr,
+                    norm_w ? f32(*norm_w, "norm_w") : nullptr, out ? out->data_ptr() : nullptr, T, ns, D, (float)eps, dy, od,
+                    cur_stream());
+}
+
+void head_linear(const Tensor& x, const Tensor& W, const optional<Tensor>& gate, Tensor& y) {
+  const int dt = act_dt(x, "x");
+  same_dt(W, dt, "W");
+  same_dt(y, dt, "y");
+  TORCH_CHECK(W.dim() == 3 && W.is_contiguous(), "head_linear: W [H, N, K] contiguous");
+  const int H = W.size(0), N = W.size(1), K = W.size(2), ldx = row_stride(x, "x"), T = x.size(0);
+  TORCH_CHECK(x.size(1) == H * K && y.is_contiguous() && y.numel() == (int64_t)T * H * N, "head_linear: shapes");
+  int ldg = 0;
+  if (gate) {
+    same_dt(*gate, dt, "gate");
+    ldg = row_stride(*gate, "gate");
+    TORCH_CHECK(gate->size(0) == T && gate->size(1) == H * N, "head_linear: gate [T, H * N]");
+  }
+  gai_head_linear(x.data_ptr(), ldx, W.data_ptr(), gate ? gate->data_ptr() : nullptr, ldg, y.data_ptr(), T, H, N, K, dt,
+                  cur_stream());
+}
+
+int64_t mlstm_ws_floats(int64_t T, int64_t S, int64_t H, int64_t DK, int64_t DV) {
+  return (int64_t)gai_mlstm_ws_floats((int)T, (int)S, (int)H, (int)DK, (int)DV);
+}
+
+void mlstm(const Tensor& q, const Tensor& k, const Tensor& v, const Tensor& ig, const Tensor& fg, const Tensor& ib,
+           const Tensor& fb, double cap, const Tensor& gate, const Tensor& norm_w, Tensor& S, Tensor& n, Tensor& m,
+           const Tensor& cu, const Tensor& slots, double q_scale, double eps, double den_eps, Tensor& y,
+           const optional<Tensor>& ws) {
+  const int dt = act_dt(q, "q");
+  same_dt(k, dt, "k");
+  same_dt(v, dt, "v");
+  same_dt(gate, dt, "gate");
+  same_dt(y, dt, "y");
+  TORCH_CHECK(S.dim() == 4, "mlstm: S [slots, H, DK, DV]");
+  const int H = S.size(1), DK = S.size(2), DV = S.size(3), T = q.size(0), nseq = slots.numel();
+  TORCH_CHECK(n.numel() == S.size(0) * H * DK && m.numel() == S.size(0) * H, "mlstm: n [slots, H, DK], m [slots, H]");
+  TORCH_CHECK(q.size(1) == H * DK && k.size(0) == T && k.size(1) == H * DK && v.size(0) == T && v.size(1) == H * DV &&
+                  gate.size(0) == T && gate.size(1) == H * DV && norm_w.numel() == H * DV && ib.numel() == H &&
+                  fb.numel() == H && cu.numel() == nseq + 1 && y.is_contiguous() && y.numel() == (int64_t)T * H * DV,
+              "mlstm: shapes");
+  TORCH_CHECK(ig.scalar_type() == at::kFloat && fg.scalar_type() == at::kFloat && ig.is_cuda() && fg.is_cuda() &&
+                  ig.size(0) == T && ig.size(1) == H && fg.size(0) == T && fg.size(1) == H, "mlstm: gate logits fp32 [T, H]");
+  float* wsp = nullptr;
+  if (ws) {
+    TORCH_CHECK(ws->is_cuda() && ws->scalar_type() == at::kFloat && ws->is_contiguous() &&
+                    ws->numel() >= mlstm_ws_floats(T, nseq, H, DK, DV), "mlstm: workspace too small");
+    wsp = ws->data_ptr<float>();
+  }
+  gai_mlstm(q.data_ptr(), row_stride(q, "q"), k.data_ptr(), row_stride(k, "k"), v.data_ptr(), row_stride(v, "v"),
+            ig.data_ptr<float>(), row_stride(ig, "ig"), fg.data_ptr<float>(), row_stride(fg, "fg"), f32(ib, "ib"),
+            f32(fb, "fb"), (float)cap, gate.data_ptr(), row_stride(gate, "gate"), f32(norm_w, "norm_w"), f32w(S, "S"),
+            f32w(n, "n"), f32w(m, "m"), i32(cu, "cu"), i32(slots, "slots"), nseq, T, H, DK, DV, (float)q_scale, (float)eps,
+            (float)den_eps, y.data_ptr(), wsp, dt, cur_stream());
+}
+
 }  // namespace
 
 void gai_bind_seq_ops(pybind11::module_& m) {
   m.def("add_dyt_f32", &add_dyt_f32);
+  m.def("latent_norm_write", &latent_norm_write);
+  m.def("hyper_connect", &hyper_connect);
+  m.def("head_linear", &head_linear);
+  m.def("mlstm", &mlstm);
+  m.def("mlstm_ws_floats", &mlstm_ws_floats);
   m.def("act_mul", &act_mul);
   m.def("latent_kv_write", &latent_kv_write);
   m.def("linear_attention_scan", &linear_attention_scan);

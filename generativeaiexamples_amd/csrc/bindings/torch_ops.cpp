@@ -498,6 +498,21 @@ void gemm_fp8(const Tensor& A, const Tensor& B, const Tensor& sa, const Tensor& 
                opt_ptr(R), M, N, K, ldc, (int)epi, f32 ? 1 : 0, (int)force, cur_stream());
 }
 
+void moe_route_chosen(const Tensor& logits, int64_t k, Tensor& ids, Tensor& w, const optional<Tensor>& bias) {
+  TORCH_CHECK(logits.is_cuda() && logits.scalar_type() == at::kFloat && logits.dim() == 2 && logits.stride(1) == 1,
+              "moe_route: logits must be fp32 GPU rows");
+  check_i32(ids, "topk ids");
+  check_f32(w, "topk weights");
+  TORCH_CHECK(ids.is_contiguous() && w.is_contiguous() && ids.numel() == logits.size(0) * k && w.numel() == ids.numel(),
+              "moe_route: ids / w [T, k]");
+  if (bias) {
+    check_f32(*bias, "router bias");
+    TORCH_CHECK(bias->is_contiguous() && bias->numel() == logits.size(1), "moe_route: bias [E]");
+  }
+  gai_moe_route_chosen(logits.data_ptr<float>(), (int)logits.stride(0), logits.size(0), logits.size(1), (int)k,
+                       ids.data_ptr<int>(), w.data_ptr<float>(), bias ? bias->data_ptr<float>() : nullptr, cur_stream());
+}
+
 void moe_route_grouped(const Tensor& logits, int64_t k, Tensor& ids, Tensor& w, const optional<Tensor>& bias, double eps,
                        int64_t groups, int64_t keep, double scale) {
   check_f32(logits, "router logits");
@@ -1013,6 +1028,7 @@ PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
   m.def("moe_route", &moe_route);
   m.def("moe_scale_rows", &moe_scale_rows);
   m.def("moe_gemm", &moe_gemm);
+  m.def("moe_route_chosen", &moe_route_chosen);
   m.def("moe_route_grouped", &moe_route_grouped);
   m.def("moe_combine", &moe_combine);
   m.def("moe_dispatch", &moe_dispatch);

@@ -147,6 +147,8 @@ void gai_moe_route(const float* logits, int T, int E, int k, int renorm, int* id
 void gai_moe_gemm(const void* A, const int* a_rows, const void* W, void* C, const int* offs, int E, int rows_total,
                   int N, int K, int act, hipStream_t st, int dt = 0, float actp = 0.f);
 // sigmoid scores, choice on score + bias among the experts of the KEEP best of NG groups, weights renormalised * scale
+void gai_moe_route_chosen(const float* logits, int ld, int T, int E, int k, int* ids, float* w, const float* bias,
+                          hipStream_t st);
 void gai_moe_route_grouped(const float* logits, int T, int E, int k, int* ids, float* w, const float* bias, float eps,
                            int NG, int KEEP, float scale, hipStream_t st);
 // w = nullptr: plain sum of the k rows
@@ -247,7 +249,24 @@ void gai_window_attention(const void* q, const void* k_cache, const void* v_cach
                           float scale, float softcap, int window, const float* r1, const float* r2, const void* gate,
                           int ldg, const float* sig_bias, int sig, float out_scale, int dt, hipStream_t st,
                           float* part = nullptr, int chunk = 0, const float* hscale = nullptr, int has_sink = 0,
-                          float sink = 0.f);
+                          float sink = 0.f, const float* hsink = nullptr);
+// q_out = rmsnorm(dq) * wq; K page row and V^T page (one kv head, key and value size R) = rmsnorm(dkv) * wkv
+void gai_latent_norm_write(const void* dq, int ldq, const float* wq, const void* dkv, int ldk, const float* wkv,
+                           const int* slots, void* q_out, void* k_cache, void* v_cache, int T, int RQ, int R, float eps,
+                           int dt, hipStream_t st);
+// hyper.hip: close one sublayer of a hyper-connected decoder (streams X, output y) and open the next (layer norm)
+void gai_hyper_connect(float* X, const float* x0, const void* y, int ldy, const float* mix, const float* out_w,
+                       const float* in_w, const float* norm_w, void* out, int T, int ns, int D, float eps, int dt_y,
+                       int dt_out, hipStream_t st);
+// head_linear.hip: y[t, h] = W[h] x[t, h] (* sigmoid(gate))
+void gai_head_linear(const void* x, int ldx, const void* W, const void* gate, int ldg, void* y, int T, int H, int N, int K,
+                     int dt, hipStream_t st);
+// mlstm.hip: scratch (fp32 elements) of a step with portions; the mixer core from projections to the gated output
+size_t gai_mlstm_ws_floats(int T, int S, int H, int DK, int DV);
+void gai_mlstm(const void* q, int ldq, const void* k, int ldk, const void* v, int ldv, const float* ig, int ldi,
+               const float* fg, int ldf, const float* ib, const float* fb, float cap, const void* gate, int ldgate,
+               const float* norm_w, float* S, float* n, float* m, const int* cu, const int* slots, int nseq, int T, int H,
+               int DK, int DV, float q_scale, float eps, float den_eps, void* y, float* ws, int dt, hipStream_t st);
 // q / k heads rotated in interleaved pairs over their first ROT channels; dt_in: input type, dt: cache / q_out type
 void gai_rotary_kv_write(const void* q, int ldq, const void* k, int ldk, const void* v, int ldv, const int* positions,
                          const int* slots, void* q_out, void* k_cache, void* v_cache, int T, int H, int G, int DK, int DV,

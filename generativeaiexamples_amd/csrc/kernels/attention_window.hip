@@ -15,8 +15,8 @@
 //
 // Chunk mode (chunk > 0): a key is visible only inside the query's own chunk of positions, floor(j / chunk) ==
 // floor(i / chunk), counted from position 0 of the sequence. hscale (per head) multiplies the scores of a head. A sink
-// (has_sink) is a virtual key of score `sink` without a value: the softmax denominator gains exp(sink). out_scale
-// multiplies the output in both modes.
+// (has_sink) is a virtual key of score `sink` (hsink: one score per head) without a value: the softmax denominator gains
+// exp(sink). out_scale multiplies the output in both modes.
 //
 // rotary_kv_write: rotation of the channel pairs (2i, 2i + 1), i < ROT / 2, of every q and k head by position *
 // base^(-2i / ROT) (the rest of a head passes unchanged), then q -> q_out and k, v -> their cache slots. The angle is
@@ -35,6 +35,9 @@
 // q_cat (whose first R channels hold the query folded through the key expansion), so window_attention scores against
 // the cached row directly. Rotation over the first ROT of the DR channels (the rest pass unchanged): channel i pairs
 // with i + ROT / 2, angle = position * inv_freq[i] (fp32, libm sincosf), cos and sin times one magnitude.
+//
+// latent_norm_write: the cache write of latent attention without rotation whose queries go through a latent of their own:
+// RMS norms of both latents in one launch, the query latent -> q_out, the key / value latent -> K page row and V^T page.
 //
 // window_attention, row kernel: one wave64 per (token, head) (a sequence is (cu_q[s], ctx[s]); the query at row t has
 // position ctx - q_len + (t - cu_q)). Keys are walked in page-aligned blocks of 64: lane j scores key j (q broadcast
@@ -242,6 +245,48 @@ __global__ __launch_bounds__(256) void latent_kv_write_kernel(const TA* __restri
   }
 }
 
+template <typename TA>
+__global__ __launch_bounds__(256) void latent_norm_write_kernel(const TA* __restrict__ dq, int ldq,
+                                                                const float* __restrict__ wq, const TA* __restrict__ dkv,
+                                                                int ldk, const float* __restrict__ wkv,
+                                                                const int* __restrict__ slots, TA* __restrict__ q_out,
+                                                                TA* __restrict__ k_cache, TA* __restrict__ v_cache, int RQ,
+                                                                int R, float eps) {
+  __shared__ float sq[4], sk[4];
+  const int t = blockIdx.x, tid = threadIdx.x;
+  const TA* qr = dq + (size_t)t * ldq;
+  const TA* kr = dkv + (size_t)t * ldk;
+  float a = 0.f, b = 0.f;
+  for (int i = tid; i < RQ; i += 256) {
+    const float x = (float)qr[i];
+    a = fmaf(x, x, a);
+  }
+  for (int i = tid; i < R; i += 256) {
+    const float x = (float)kr[i];
+    b = fmaf(x, x, b);
+  }
+  a = wave_sum(a);
+  b = wave_sum(b);
+  if ((tid & 63) == 0) {
+    sq[tid >> 6] = a;
+    sk[tid >> 6] = b;
+  }
+  __syncthreads();
+  const float iq = 1.0f / sqrtf((sq[0] + sq[1] + sq[2] + sq[3]) / RQ + eps);
+  const float ik = 1.0f / sqrtf((sk[0] + sk[1] + sk[2] + sk[3]) / R + eps);
+  TA* qo = q_out + (size_t)t * RQ;
+  for (int i = tid; i < RQ; i += 256) qo[i] = (TA)((float)qr[i] * iq * wq[i]);
+  const int slot = slots[t];
+  const size_t page = slot >> 4;
+  const int off = slot & 15;
+  TA* kp = k_cache + (page * 16 + off) * R;
+  for (int i = tid; i < R; i += 256) {
+    const TA c = (TA)((float)kr[i] * ik * wkv[i]);
+    kp[i] = c;
+    v_cache[(page * R + i) * 16 + off] = c;
+  }
+}
+
 template <typename TI, typename TA>
 __global__ __launch_bounds__(256) void rotary_kv_write_kernel(const TI* __restrict__ q, int ldq, const TI* __restrict__ k,
                                                               int ldk, const TI* __restrict__ v, int ldv,
@@ -309,7 +354,7 @@ __global__ __launch_bounds__(256) void window_attention_kernel(
     TA* __restrict__ out, int ldo, int TH, int H, int G, int DK, int DV, float scale, float softcap, int window,
     const float* __restrict__ r1, const float* __restrict__ r2, const TA* __restrict__ gate, int ldg, int skip_len,
     const float* __restrict__ sig_bias, float out_scale, int nsplit, float* __restrict__ part, int chunk,
-    const float* __restrict__ hscale, int has_sink, float sink) {
+    const float* __restrict__ hscale, int has_sink, float sink, const float* __restrict__ hsink) {
   extern __shared__ float lds[];
   const int wid = threadIdx.x >> 6, lane = threadIdx.x & 63;
   const int th = blockIdx.x * 4 + wid;
@@ -328,6 +373,7 @@ __global__ __launch_bounds__(256) void window_attention_kernel(
   int first = window > 0 ? max(0, pos - window + 1) : 0;
   if (chunk > 0) first = max(first, pos / chunk * chunk);
   if (hscale) scale *= hscale[h];
+  if (hsink) sink = hsink[h];
   const TA* qr = q + (size_t)th * DK;
   for (int i = lane; i < DK; i += 64) qs[i] = (float)qr[i];
   __builtin_amdgcn_wave_barrier();
@@ -435,11 +481,13 @@ template <typename TA>
 __global__ __launch_bounds__(256) void softmax_split_reduce_kernel(const float* __restrict__ part, int nsplit,
                                                                    TA* __restrict__ out, int ldo, int T, int H, int DV,
                                                                    const TA* __restrict__ gate, int ldg, float out_scale,
-                                                                   int has_sink, float sink) {
+                                                                   int has_sink, float sink,
+                                                                   const float* __restrict__ hsink) {
   const long e = (long)blockIdx.x * 256 + threadIdx.x;
   if (e >= (long)T * H * DV) return;
   const int th = (int)(e / DV), c = (int)(e % DV), t = th / H, h = th - t * H;
   const size_t TH = (size_t)T * H, W = DV + 2;
+  if (hsink) sink = hsink[h];
   float M = has_sink ? sink : -INFINITY;
   for (int sp = 0; sp < nsplit; ++sp) M = fmaxf(M, part[((size_t)sp * TH + th) * W + DV]);
   float num = 0.f, den = has_sink ? expf(sink - M) : 0.f;
@@ -491,11 +539,13 @@ __global__ __launch_bounds__(256) void window_attention_mfma_kernel(
     const int* __restrict__ block_tables, int maxb, const int* __restrict__ cu_q, const int* __restrict__ ctx, int S,
     bf16* __restrict__ out, int ldo, int H, int G, float scale, float softcap, int window, const float* __restrict__ r1,
     const float* __restrict__ r2, const bf16* __restrict__ gate, int ldg, const float* __restrict__ sig_bias,
-    float out_scale, int chunk, const float* __restrict__ hscale, int has_sink, float sink) {
+    float out_scale, int chunk, const float* __restrict__ hscale, int has_sink, float sink,
+    const float* __restrict__ hsink) {
   const int wid = threadIdx.x >> 6, lane = threadIdx.x & 63;
   const int h = blockIdx.y * 4 + wid;
   if (h >= H) return;
   if (hscale) scale *= hscale[h];
+  if (hsink) sink = hsink[h];
   // tile -> (sequence, first row): sequences of at least kMfmaMinLen rows own ceil(len / 32) tiles each
   int s = 0, seen = 0, len = 0;
   for (; s < S; ++s) {
@@ -624,16 +674,17 @@ void launch_window_mfma(const void* q, const void* k_cache, const void* v_cache,
                         const int* cu_q, const int* ctx, int S, void* out, int ldo, int T, int H, int G, float scale,
                         float softcap, int window, const float* r1, const float* r2, const void* gate, int ldg,
                         const float* sig_bias, int sig, float out_scale, hipStream_t st, int chunk, const float* hscale,
-                        int has_sink, float sink) {
+                        int has_sink, float sink, const float* hsink) {
   const dim3 grid((T + kTileQ - 1) / kTileQ + S, (H + 3) / 4);
   if (sig)
     window_attention_mfma_kernel<DK, DV, true><<<grid, 256, 0, st>>>(
         (const bf16*)q, (const bf16*)k_cache, (const bf16*)v_cache, block_tables, maxb, cu_q, ctx, S, (bf16*)out, ldo, H,
-        G, scale, softcap, window, r1, r2, (const bf16*)gate, ldg, sig_bias, out_scale, chunk, hscale, has_sink, sink);
+        G, scale, softcap, window, r1, r2, (const bf16*)gate, ldg, sig_bias, out_scale, chunk, hscale, has_sink, sink, hsink);
   else
     window_attention_mfma_kernel<DK, DV, false><<<grid, 256, 0, st>>>(
         (const bf16*)q, (const bf16*)k_cache, (const bf16*)v_cache, block_tables, maxb, cu_q, ctx, S, (bf16*)out, ldo, H,
-        G, scale, softcap, window, r1, r2, (const bf16*)gate, ldg, sig_bias, out_scale, chunk, hscale, has_sink, sink);
+        G, scale, softcap, window, r1, r2, (const bf16*)gate, ldg, sig_bias, out_scale, chunk, hscale, has_sink, sink,
+        hsink);
 }
 
 }  // namespace
@@ -688,6 +739,19 @@ void gai_latent_kv_write(const void* q, int ldq, const void* dkv, int ldk, const
   GAI_LAUNCH_CHECK();
 }
 
+void gai_latent_norm_write(const void* dq, int ldq, const float* wq, const void* dkv, int ldk, const float* wkv,
+                           const int* slots, void* q_out, void* k_cache, void* v_cache, int T, int RQ, int R, float eps,
+                           int dt, hipStream_t st) {
+  if (T == 0) return;
+  if (dt)
+    latent_norm_write_kernel<float><<<T, 256, 0, st>>>((const float*)dq, ldq, wq, (const float*)dkv, ldk, wkv, slots,
+                                                       (float*)q_out, (float*)k_cache, (float*)v_cache, RQ, R, eps);
+  else
+    latent_norm_write_kernel<bf16><<<T, 256, 0, st>>>((const bf16*)dq, ldq, wq, (const bf16*)dkv, ldk, wkv, slots,
+                                                      (bf16*)q_out, (bf16*)k_cache, (bf16*)v_cache, RQ, R, eps);
+  GAI_LAUNCH_CHECK();
+}
+
 // dt_in / dt: 0 = bf16, 1 = fp32 (inputs may be fp32 while the cache is bf16: the output of an fp32 convolution)
 void gai_rotary_kv_write(const void* q, int ldq, const void* k, int ldk, const void* v, int ldv, const int* positions,
                          const int* slots, void* q_out, void* k_cache, void* v_cache, int T, int H, int G, int DK, int DV,
@@ -716,8 +780,9 @@ void gai_window_attention(const void* q, const void* k_cache, const void* v_cach
                           const int* cu_q, const int* ctx, int S, void* out, int ldo, int T, int H, int G, int DK, int DV,
                           float scale, float softcap, int window, const float* r1, const float* r2, const void* gate,
                           int ldg, const float* sig_bias, int sig, float out_scale, int dt, hipStream_t st,
-                          float* part, int chunk, const float* hscale, int has_sink, float sink) {
+                          float* part, int chunk, const float* hscale, int has_sink, float sink, const float* hsink) {
   if (T == 0 || S == 0) return;
+  if (hsink) has_sink = 1;
   if (sig && (chunk > 0 || hscale || has_sink))
     gai_launch_error(__FILE__, __LINE__, "window_attention: chunks, head scales and sinks go with the softmax mode");
   if (DV > 64 * kMaxVChunks) gai_launch_error(__FILE__, __LINE__, "window_attention: value head size above 512");
@@ -732,12 +797,14 @@ void gai_window_attention(const void* q, const void* k_cache, const void* v_cach
   if (DK == K_ && DV == V_) {                                                                                        \
     launch_window_mfma<K_, V_>(q, k_cache, v_cache, block_tables, maxb, cu_q, ctx, S, out, ldo, T, H, G, scale,      \
                                softcap, window, r1, r2, gate, ldg, sig_bias, sig, out_scale, st, chunk, hscale,       \
-                               has_sink, sink);                                                                      \
+                               has_sink, sink, hsink);                                                               \
     skip_len = kMfmaMinLen;                                                                                          \
   }
     GAI_WIN(64, 64) GAI_WIN(64, 128) GAI_WIN(128, 64) GAI_WIN(128, 128) GAI_WIN(256, 256)
     // latent rows: key row = latent + rotated part, value row = latent
     GAI_WIN(96, 64) GAI_WIN(192, 128) GAI_WIN(320, 256)
+    // latent rows without a rotated part
+    GAI_WIN(32, 32) GAI_WIN(96, 96) GAI_WIN(160, 160) GAI_WIN(192, 192)
 #undef GAI_WIN
     GAI_LAUNCH_CHECK();
   }
@@ -746,7 +813,7 @@ void gai_window_attention(const void* q, const void* k_cache, const void* v_cach
   window_attention_kernel<TA, SIG_><<<dim3(grid, nsplit), 256, lds, st>>>(                                           \
       (const TA*)q, (const TA*)k_cache, (const TA*)v_cache, block_tables, maxb, cu_q, ctx, S, (TA*)out, ldo, TH, H, G, \
       DK, DV, scale, softcap, window, r1, r2, (const TA*)gate, ldg, skip_len, sig_bias, out_scale, nsplit, part,    \
-      chunk, hscale, has_sink, sink)
+      chunk, hscale, has_sink, sink, hsink)
   if (dt) {
     if (sig) GAI_ROW(float, true); else GAI_ROW(float, false);
   } else {
@@ -758,11 +825,11 @@ void gai_window_attention(const void* q, const void* k_cache, const void* v_cach
     if (dt)
       softmax_split_reduce_kernel<float><<<(unsigned)((n + 255) / 256), 256, 0, st>>>(part, nsplit, (float*)out, ldo, T, H,
                                                                                        DV, (const float*)gate, ldg,
-                                                                                       out_scale, has_sink, sink);
+                                                                                       out_scale, has_sink, sink, hsink);
     else
       softmax_split_reduce_kernel<bf16><<<(unsigned)((n + 255) / 256), 256, 0, st>>>(part, nsplit, (bf16*)out, ldo, T, H,
                                                                                       DV, (const bf16*)gate, ldg,
-                                                                                      out_scale, has_sink, sink);
+                                                                                      out_scale, has_sink, sink, hsink);
   } else if (nsplit > 1) {
     const long n = (long)T * H * DV;
     if (dt)

@@ -19,6 +19,8 @@
 // moe_combine (identity experts): a chosen id >= n_real has no weights - its output is the token's own input row.
 // moe_route (grouped sigmoid): choice on sigmoid score + bias confined to the best contiguous expert groups (ranked by their
 //              top-2 choice scores added up); weights = the chosen plain scores renormalised (+ eps), scaled.
+// moe_route (chosen): bias is part of the logits; the top-k logits + bias are chosen and weighted by the softmax over the
+//              chosen ones only; libm expf, all fp32.
 // moe_gemm (clamped gated): g = min(gate, p), u = clamp(up, +-p), g sigmoid(1.702 g) (u + 1) on [gate16 | up16] rows.
 // moe_combine (residual gate): the residual row (a shared expert's output) times sigmoid of a per-token logit.
 // moe_scale_rows: expert-sorted copies of the token rows, each times its routing weight (experts whose routing weight
@@ -75,6 +77,40 @@ __global__ void moe_route_kernel(const float* __restrict__ logits, int T, int E,
   for (int j = 0; j < k; ++j) {
     ids[(size_t)t * k + j] = bi[j];
     w[(size_t)t * k + j] = (renorm && !sigmoid) ? bv[j] / tot : bv[j];
+  }
+}
+
+// ld: row stride of the logits (a column slice of a padded projection)
+__global__ void moe_route_chosen_kernel(const float* __restrict__ logits, int ld, int T, int E, int k,
+                                        int* __restrict__ ids, float* __restrict__ w, const float* __restrict__ bias) {
+  const int t = blockIdx.x * blockDim.x + threadIdx.x;
+  if (t >= T) return;
+  const float* x = logits + (size_t)t * ld;
+  float bv[16];
+  int bi[16];
+  for (int j = 0; j < k; ++j) { bv[j] = -INFINITY; bi[j] = -1; }
+  for (int e = 0; e < E; ++e) {
+    const float z = x[e] + (bias ? bias[e] : 0.f);
+    if (z > bv[k - 1] || bi[k - 1] < 0) {
+      int j = k - 1;
+      while (j > 0 && (bi[j - 1] < 0 || bv[j - 1] < z)) {
+        bv[j] = bv[j - 1];
+        bi[j] = bi[j - 1];
+        --j;
+      }
+      bv[j] = z;
+      bi[j] = e;
+    }
+  }
+  float tot = 0.f;
+  const float mx = bv[0];
+  for (int j = 0; j < k; ++j) {
+    bv[j] = expf(bv[j] - mx);
+    tot += bv[j];
+  }
+  for (int j = 0; j < k; ++j) {
+    ids[(size_t)t * k + j] = bi[j];
+    w[(size_t)t * k + j] = bv[j] / tot;
   }
 }
 
@@ -576,6 +612,14 @@ void gai_moe_scale_rows(const void* h, const int* pos, const float* w, void* out
     moe_scale_rows_kernel<float><<<T * k, 256, 0, st>>>((const float*)h, pos, w, (float*)out, k, D);
   else
     moe_scale_rows_kernel<bf16><<<T * k, 256, 0, st>>>((const bf16*)h, pos, w, (bf16*)out, k, D);
+  GAI_LAUNCH_CHECK();
+}
+
+void gai_moe_route_chosen(const float* logits, int ld, int T, int E, int k, int* ids, float* w, const float* bias,
+                          hipStream_t st) {
+  if (T == 0) return;
+  if (k < 1 || k > 16 || k > E) gai_launch_error(__FILE__, __LINE__, "moe_route: 1 <= top-k <= min(16, experts)");
+  moe_route_chosen_kernel<<<(T + 63) / 64, 64, 0, st>>>(logits, ld, T, E, k, ids, w, bias);
   GAI_LAUNCH_CHECK();
 }
 
