@@ -6,7 +6,7 @@ Architecture (every size and constant comes from ``config.json``; the layer list
   * ``streams`` residual streams X_1 .. X_s, all equal to the embedding output at first. A sublayer (mixer, feed-forward) reads
     ``u = sum_s in[s] X_s`` through a layer norm (weight, no bias) and its output y goes back as
     ``X_t <- sum_s mix[s, t] X_s + out[t] y``; after the last layer the streams are summed;
-  * a layer may have no feed-forward, and may use the weights of an earlier one (``weights_of``) with a cache / state of its
+  * a layer may have no feed-forward, and may use the weights of another one (``weights_of``) with a cache / state of its
     own;
   * mixer ``latent_attention``: queries from a normed low-rank latent of their own, keys and values linear maps of one normed
     latent per token (all of the cache), no positions, causal softmax with a learned value-less sink score per head, the
@@ -76,14 +76,14 @@ class LuketarConfig:
                     raise ValueError(f"layer {i}: unknown feed-forward kind {kind!r}")
                 if kind == "moe" and not 1 <= ml["router"]["top"] <= min(16, ml["router"]["experts"]):
                     raise ValueError(f"layer {i}: 1 <= top <= min(16, experts)")
-            j = l.get("weights_of")
-            if j is not None:
-                if not 0 <= j < i:
-                    raise ValueError(f"layer {i}: weights_of names an earlier layer")
-                if layers[j]["type"] != l["type"] or layers[j]["mixer"] != m or layers[j]["mlp"] != ml:
-                    raise ValueError(f"layer {i}: differs from layer {j}, whose weights it uses")
             layers.append(dict(l, mixer=m, mlp=ml))
         self.layers = tuple(layers)
+        for i, l in enumerate(layers):
+            if l.get("weights_of") is None:
+                continue
+            j = self.weight_layer(i)
+            if layers[j]["type"] != l["type"] or layers[j]["mixer"] != l["mixer"] or layers[j]["mlp"] != l["mlp"]:
+                raise ValueError(f"layer {i}: differs from layer {j}, whose weights it uses")
 
     @property
     def num_layers(self) -> int:
@@ -95,9 +95,12 @@ class LuketarConfig:
 
     def weight_layer(self, i: int) -> int:
         """The layer whose tensors layer i uses."""
-        while self.layers[i].get("weights_of") is not None:
-            i = self.layers[i]["weights_of"]
-        return i
+        j, hops = i, 0
+        while self.layers[j].get("weights_of") is not None:
+            j, hops = int(self.layers[j]["weights_of"]), hops + 1
+            if not 0 <= j < len(self.layers) or hops > len(self.layers):
+                raise ValueError(f"layer {i}: weights_of does not lead to a layer with weights of its own")
+        return j
 
     @staticmethod
     def from_json(path_or_dict) -> "LuketarConfig":
