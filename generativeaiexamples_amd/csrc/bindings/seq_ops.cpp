@@ -557,6 +557,33 @@ void selective_scan(const Tensor& x, const Tensor& dt, const Tensor& dt_bias, co
                      I, N, dtt, cur_stream());
 }
 
+int64_t mqa_attention_ws_floats(int64_t T, int64_t S, int64_t H, int64_t DV) {
+  return (int64_t)gai_mqa_attention_ws_floats((int)T, (int)S, (int)H, (int)DV);
+}
+
+void mqa_attention(const Tensor& q, const Tensor& k_cache, const Tensor& v_cache, const Tensor& block_tables,
+                   const Tensor& cu_q, const Tensor& ctx, Tensor& out, int64_t H, double scale, int64_t window,
+                   const optional<Tensor>& sink, const optional<Tensor>& ws) {
+  TORCH_CHECK(act_dt(q, "q") == 0 && act_dt(out, "out") == 0, "mqa_attention: bf16");
+  const int DK = k_cache.size(3), DV = v_cache.size(2), S = ctx.numel();
+  check_cache(k_cache, v_cache, 0, 1, DK, DV);
+  TORCH_CHECK(gai_mqa_attention_ok(DK, DV), "mqa_attention: no kernel for these key / value sizes");
+  TORCH_CHECK(q.is_contiguous() && q.numel() % (H * DK) == 0, "mqa_attention: q shape");
+  const int T = q.numel() / (H * DK), ldo = row_stride(out, "out");
+  TORCH_CHECK(out.size(0) == T && out.size(1) == H * DV && cu_q.numel() == S + 1 && block_tables.dim() == 2 &&
+                  block_tables.size(0) >= S, "mqa_attention: out / cu_q / block table shapes");
+  TORCH_CHECK(((size_t)out.data_ptr() & 7) == 0 && ldo % 4 == 0, "mqa_attention: output rows on a grid of four elements");
+  if (sink) TORCH_CHECK(sink->numel() == H, "mqa_attention: one sink score per head");
+  const int64_t need = mqa_attention_ws_floats(T, S, H, DV);
+  if (need)
+    TORCH_CHECK(ws && ws->is_cuda() && ws->scalar_type() == at::kFloat && ws->is_contiguous() && ws->numel() >= need,
+                "mqa_attention: workspace too small");
+  gai_mqa_attention(q.data_ptr(), k_cache.data_ptr(), v_cache.data_ptr(), i32(block_tables, "block_tables"),
+                    block_tables.size(1), i32(cu_q, "cu_q"), i32(ctx, "ctx"), S, out.data_ptr(), ldo, T, (int)H, DK, DV,
+                    (float)scale, (int)window, sink ? f32(*sink, "sink") : nullptr, need ? ws->data_ptr<float>() : nullptr,
+                    cur_stream());
+}
+
 void latent_norm_write(const Tensor& dq, const Tensor& wq, const Tensor& dkv, const Tensor& wkv, const Tensor& slots,
                        Tensor& q_out, Tensor& k_cache, Tensor& v_cache, double eps) {
   const int dt = act_dt(dq, "dq");
@@ -653,6 +680,9 @@ void mlstm(const Tensor& q, const Tensor& k, const Tensor& v, const Tensor& ig, 
 
 void gai_bind_seq_ops(pybind11::module_& m) {
   m.def("add_dyt_f32", &add_dyt_f32);
+  m.def("mqa_attention", &mqa_attention);
+  m.def("mqa_attention_ok", [](int64_t DK, int64_t DV) { return gai_mqa_attention_ok((int)DK, (int)DV) != 0; });
+  m.def("mqa_attention_ws_floats", &mqa_attention_ws_floats);
   m.def("latent_norm_write", &latent_norm_write);
   m.def("hyper_connect", &hyper_connect);
   m.def("head_linear", &head_linear);

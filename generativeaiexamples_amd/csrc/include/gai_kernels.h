@@ -254,6 +254,12 @@ void gai_window_attention(const void* q, const void* k_cache, const void* v_cach
 void gai_latent_norm_write(const void* dq, int ldq, const float* wq, const void* dkv, int ldk, const float* wkv,
                            const int* slots, void* q_out, void* k_cache, void* v_cache, int T, int RQ, int R, float eps,
                            int dt, hipStream_t st);
+// attention_mqa.hip: bf16 softmax attention with one kv head shared by all heads, optional window and sinks per head
+int gai_mqa_attention_ok(int DK, int DV);
+size_t gai_mqa_attention_ws_floats(int T, int S, int H, int DV);
+void gai_mqa_attention(const void* q, const void* k_cache, const void* v_cache, const int* block_tables, int maxb,
+                       const int* cu_q, const int* ctx, int S, void* out, int ldo, int T, int H, int DK, int DV, float scale,
+                       int window, const float* sink, float* ws, hipStream_t st);
 // hyper.hip: close one sublayer of a hyper-connected decoder (streams X, output y) and open the next (layer norm)
 void gai_hyper_connect(float* X, const float* x0, const void* y, int ldy, const float* mix, const float* out_w,
                        const float* in_w, const float* norm_w, void* out, int T, int ns, int D, float eps, int dt_y,

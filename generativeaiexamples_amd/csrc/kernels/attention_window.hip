@@ -803,8 +803,6 @@ void gai_window_attention(const void* q, const void* k_cache, const void* v_cach
     GAI_WIN(64, 64) GAI_WIN(64, 128) GAI_WIN(128, 64) GAI_WIN(128, 128) GAI_WIN(256, 256)
     // latent rows: key row = latent + rotated part, value row = latent
     GAI_WIN(96, 64) GAI_WIN(192, 128) GAI_WIN(320, 256)
-    // latent rows without a rotated part
-    GAI_WIN(32, 32) GAI_WIN(96, 96) GAI_WIN(160, 160) GAI_WIN(192, 192)
 #undef GAI_WIN
     GAI_LAUNCH_CHECK();
   }

@@ -1201,11 +1201,19 @@ def window_attention(q, k_cache, v_cache, block_tables, cu_q, ctx, H: int, G: in
                                                softcap, window, r1, r2, gate))
     if out is None:
         out = torch.empty(q.shape[0], H * DV, dtype=q.dtype, device=q.device)
+    hs = sink if isinstance(sink, torch.Tensor) else None
+    if (G == 1 and q.dtype == torch.bfloat16 and not softcap and r1 is None and gate is None and not chunk
+            and head_scale is None and out_scale == 1.0 and (sink is None or hs is not None)
+            and native().mqa_attention_ok(DK, DV)):
+        # one kv head: (token, head) rows share the keys, so tiles mix heads and tokens (attention_mqa.hip)
+        n = native().mqa_attention_ws_floats(q.shape[0], ctx.numel(), H, DV)
+        ws = torch.empty(n, dtype=torch.float32, device=q.device) if n else None
+        native().mqa_attention(q, k_cache, v_cache, block_tables, cu_q, ctx, out, H, float(scale), int(window or 0), hs, ws)
+        return out
     # decode steps of few rows: the keys of a row are split over several waves, merged from (sums, maximum, denominator)
     T, S = q.shape[0], ctx.numel()
     ns = native().sigmoid_attention_splits(T, S, H)
     part = torch.empty(ns * T * H * (DV + 2), dtype=torch.float32, device=q.device) if ns > 1 else None
-    hs = sink if isinstance(sink, torch.Tensor) else None
     native().window_attention(q, k_cache, v_cache, block_tables, cu_q, ctx, out, H, G, DK, DV, float(scale),
                               float(softcap or 0.0), int(window or 0), r1, r2, gate, None, False, float(out_scale), part,
                               int(chunk or 0), head_scale, None if sink is None or hs is not None else float(sink), hs)
