@@ -40,6 +40,7 @@ struct MqaArgs {
   int ldo;
   float* part;                     // [nsplit][T * H][DV + 4]: sums, maximum (log2 units), denominator
   int nsplit;
+  int tps;                         // tiles of 32 rows per sequence in the key-split launch
 };
 
 __device__ __forceinline__ int key_perm(int i) { return (i & 0x13) | ((i & 4) << 1) | ((i & 8) >> 1); }
@@ -215,11 +216,11 @@ __global__ __launch_bounds__(64 * NW) void mqa_prefill_kernel(MqaArgs a) {
     }
 }
 
-// blockIdx.x = sequence * 4 + tile of 32 rows, blockIdx.y = share of the key blocks
+// blockIdx.x = sequence * tps + tile of 32 rows, blockIdx.y = share of the key blocks
 template <int DK, int DV>
 __global__ __launch_bounds__(64) void mqa_split_kernel(MqaArgs a) {
   const int lane = threadIdx.x, qi = lane & 31, hb = lane >> 5;
-  const int s = blockIdx.x >> 2, r0 = (blockIdx.x & 3) * 32;
+  const int s = blockIdx.x / a.tps, r0 = (blockIdx.x % a.tps) * 32;
   const int len = a.cu[s + 1] - a.cu[s], rows = len * a.H;
   if (rows >= kShortRows || r0 >= rows) return;
   const int c0 = a.ctx[s] - len, row = min(r0 + qi, rows - 1);
@@ -234,13 +235,7 @@ __global__ __launch_bounds__(64) void mqa_split_kernel(MqaArgs a) {
   float* po = a.part + ((size_t)blockIdx.y * a.T * a.H + g_row) * (DV + 4);
   const bool mine = r0 + qi < rows;
   float m = kOut, l = 0.f;
-  if (kb0 > kb1) {  // no key block left for this share
-    if (mine && hb == 0) {
-      po[DV] = m;
-      po[DV + 1] = l;
-    }
-    return;
-  }
+  if (kb0 > kb1) return;  // no key block left for this share: the merge does not read it
   const bf16* qr = a.q + g_row * DK + 8 * hb;
   bf16x8 qf[DK / 16];
 #pragma unroll
@@ -252,20 +247,25 @@ __global__ __launch_bounds__(64) void mqa_split_kernel(MqaArgs a) {
   for (int kb = kb0; kb <= kb1; kb += 32) {
     const int pg[2] = {bt[kb >> 4], bt[min((kb >> 4) + 1, lp)]};
     const bf16* kp = a.kc + ((size_t)(kr < 16 ? pg[0] : pg[1]) * 16 + (kr & 15)) * DK + 8 * hb;
+    bf16x8 kf[DK / 16], vf[2][DV / 32];  // the values of the block are on their way while it is scored
+#pragma unroll
+    for (int i = 0; i < DK / 16; ++i) kf[i] = load8(kp + 16 * i);
+#pragma unroll
+    for (int k2 = 0; k2 < 2; ++k2)
+#pragma unroll
+      for (int i = 0; i < DV / 32; ++i) vf[k2][i] = load8(a.vc + ((size_t)pg[k2] * DV + qi) * 16 + 8 * hb + 32 * i * 16);
     f32x16 sc = f32x16{};
 #pragma unroll
-    for (int i = 0; i < DK / 16; ++i) sc = __builtin_amdgcn_mfma_f32_32x32x16_bf16(load8(kp + 16 * i), qf[i], sc, 0, 0, 0);
+    for (int i = 0; i < DK / 16; ++i) sc = __builtin_amdgcn_mfma_f32_32x32x16_bf16(kf[i], qf[i], sc, 0, 0, 0);
     soft_block(sc, a.scale2, kb + 31 > p_first || kb < lo_last, kb, pos, lo, hb, m, l, acc);
 #pragma unroll
     for (int k2 = 0; k2 < 2; ++k2) {
       bf16x8 ph, pl;
       split_weights(sc, k2, ph, pl);
-      const bf16* vp = a.vc + ((size_t)pg[k2] * DV + qi) * 16 + 8 * hb;
 #pragma unroll
       for (int i = 0; i < DV / 32; ++i) {
-        const bf16x8 vf = load8(vp + (size_t)32 * i * 16);
-        acc[i] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(vf, ph, acc[i], 0, 0, 0);
-        acc[i] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(vf, pl, acc[i], 0, 0, 0);
+        acc[i] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(vf[k2][i], ph, acc[i], 0, 0, 0);
+        acc[i] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(vf[k2][i], pl, acc[i], 0, 0, 0);
       }
     }
   }
@@ -283,18 +283,23 @@ __global__ __launch_bounds__(64) void mqa_split_kernel(MqaArgs a) {
   }
 }
 
-// one wave per row of the short sequences: blockIdx.x = sequence * kShortRows + row
+// one wave per row (blockIdx.x) of every short sequence (blockIdx.y)
 template <int DV>
 __global__ __launch_bounds__(64) void mqa_merge_kernel(MqaArgs a) {
   __shared__ float wgt[kMaxSplit];
-  const int s = blockIdx.x / kShortRows, row = blockIdx.x % kShortRows, lane = threadIdx.x;
+  const int s = blockIdx.y, row = blockIdx.x, lane = threadIdx.x;
   const int rows = (a.cu[s + 1] - a.cu[s]) * a.H;
   if (rows >= kShortRows || row >= rows) return;
   const size_t g_row = (size_t)a.cu[s] * a.H + row, TH = (size_t)a.T * a.H;
   const float* p0 = a.part + g_row * (DV + 4);
   const size_t step = TH * (DV + 4);
+  // the shares that held key blocks of this row's tile, as the key-split kernel dealt them out
+  const int len = a.cu[s + 1] - a.cu[s], c0 = a.ctx[s] - len, r0 = row & ~31;
+  const int k_lo = (a.window > 0 ? max(0, c0 + r0 / a.H - a.window + 1) : 0) & ~31;
+  const int nblk = (c0 + min(r0 + 31, rows - 1) / a.H - k_lo) / 32 + 1, per = (nblk + a.nsplit - 1) / a.nsplit;
+  const int used = (nblk + per - 1) / per;
   float m = kOut, l = 0.f;
-  if (lane < a.nsplit) {
+  if (lane < used) {
     m = p0[lane * step + DV];
     l = p0[lane * step + DV + 1];
   }
@@ -302,23 +307,22 @@ __global__ __launch_bounds__(64) void mqa_merge_kernel(MqaArgs a) {
   const float M = fmaxf(wave_max(m), sk);
   const float w = l > 0.f ? __builtin_amdgcn_exp2f(m - M) : 0.f;
   const float den = wave_sum(l * w) + (a.sink ? __builtin_amdgcn_exp2f(sk - M) : 0.f);
-  if (lane < a.nsplit) wgt[lane] = w / den;
+  if (lane < used) wgt[lane] = w / den;
   __syncthreads();
   const int t = a.cu[s] + row / a.H;
   bf16* o = a.out + (size_t)t * a.ldo + (size_t)(row % a.H) * DV;
   for (int c = 4 * lane; c < DV; c += 256) {
     f32x4 y = f32x4{0.f, 0.f, 0.f, 0.f};
 #pragma unroll 8
-    for (int j = 0; j < a.nsplit; ++j) {
-      const float wj = wgt[j];
-      if (wj != 0.f) y += wj * *reinterpret_cast<const f32x4*>(p0 + j * step + c);  // a share without keys wrote no sums
-    }
+    for (int j = 0; j < used; ++j) y += wgt[j] * *reinterpret_cast<const f32x4*>(p0 + j * step + c);
     *reinterpret_cast<bf16x4*>(o + c) = bf16x4{(bf16)y[0], (bf16)y[1], (bf16)y[2], (bf16)y[3]};
   }
 }
 
+int tiles_per_seq(int T, int S, int H) { return T == S ? (H + 31) / 32 : kShortRows / 32; }
+
 int split_count(int T, int S, int H) {
-  const int tiles = S * ((min(T / S, 4) * H + 31) / 32);
+  const int tiles = S * (T == S ? (H + 31) / 32 : (T / S < 4 ? T / S * H + 31 : kShortRows) / 32);
   int n = 1024 / (tiles < 1 ? 1 : tiles);
   return n < 4 ? 4 : (n > kMaxSplit ? kMaxSplit : n);
 }
@@ -342,8 +346,8 @@ void launch(const MqaArgs& a, hipStream_t st) {
     }
   }
   if (a.H < kShortRows) {
-    mqa_split_kernel<DK, DV><<<dim3(4 * a.S, a.nsplit), 64, 0, st>>>(a);
-    mqa_merge_kernel<DV><<<kShortRows * a.S, 64, 0, st>>>(a);
+    mqa_split_kernel<DK, DV><<<dim3(a.tps * a.S, a.nsplit), 64, 0, st>>>(a);
+    mqa_merge_kernel<DV><<<dim3(32 * a.tps, a.S), 64, 0, st>>>(a);
   }
 }
 
@@ -365,7 +369,7 @@ void gai_mqa_attention(const void* q, const void* k_cache, const void* v_cache, 
   if (T == 0 || S == 0) return;
   if (ldo % 4) gai_launch_error(__FILE__, __LINE__, "mqa_attention: output rows on a grid of four elements");
   const MqaArgs a{(const bf16*)q, (const bf16*)k_cache, (const bf16*)v_cache, block_tables, cu_q, ctx, maxb, S, T, H,
-                  scale * kL2e, window, sink, (bf16*)out, ldo, ws, split_count(T, S, H)};
+                  scale * kL2e, window, sink, (bf16*)out, ldo, ws, split_count(T, S, H), tiles_per_seq(T, S, H)};
   if (H < kShortRows && !ws) gai_launch_error(__FILE__, __LINE__, "mqa_attention: scratch missing");
 #define GAI_MQA(K_, V_) if (DK == K_ && DV == V_) { launch<K_, V_>(a, st); GAI_LAUNCH_CHECK(); return; }
   GAI_MQA(32, 32) GAI_MQA(64, 64) GAI_MQA(96, 96) GAI_MQA(128, 128) GAI_MQA(160, 160) GAI_MQA(192, 192) GAI_MQA(256, 256)

@@ -11,6 +11,9 @@
 //              the fused w1|w3 projection.
 //              act: SwiGLU or squared ReLU in the epilogue. fp32 operands and K off the 64 grid run on a generic
 //              LDS-tiled grouped kernel with fp32 FMA (true fp32 arithmetic).
+//              Decode-sized steps whose K does not fit the LDS-staged weight stream (gemm_decode.hip) run
+//              moe_gemm_stream: workgroups of 8 waves split K for 16 RT output channels of one expert, weight fragments
+//              straight from memory into v_mfma_f32_16x16x32_bf16 (16 token rows per column tile), partial sums added in LDS.
 // moe_combine: out[t] = sum_j w[t, j] * Y[pos[t, j]] (+ residual), bf16x8 vectorised (generic kernel: fp32 rows, any
 //              width, w optional).
 // moe_route (sigmoid): every expert scored alone by sigmoid(logit); the weights are the chosen scores.
@@ -634,6 +637,100 @@ void gai_moe_route_grouped(const float* logits, int T, int E, int k, int* ids, f
   GAI_LAUNCH_CHECK();
 }
 
+// decode-sized grouped GEMM as a weight stream for any K % 32 == 0: see the head of this file
+template <int ACT, int RT, int MB>
+static __global__ __launch_bounds__(512) void moe_gemm_stream_kernel(const bf16* __restrict__ A, const int* __restrict__ a_rows,
+                                                              const bf16* __restrict__ W, bf16* __restrict__ C,
+                                                              const int* __restrict__ offs, int N, int K, float actp) {
+  __shared__ __attribute__((aligned(16))) float red[8][RT * MB][256];
+  const int e = blockIdx.y, r_lo = offs[e], cnt = offs[e + 1] - r_lo;
+  if (cnt <= 0) return;
+  const int tid = threadIdx.x, wv = tid >> 6, lane = tid & 63, ri = lane & 15, g = lane >> 4;
+  const int n0 = blockIdx.x * 16 * RT;
+  const int steps = K / 32, per = (steps + 7) / 8, s0 = min(steps, wv * per), s1 = min(steps, s0 + per);
+  const bf16* w = W + ((size_t)e * N + n0 + ri) * K + 8 * g;
+  for (int c0 = 0; c0 < cnt; c0 += 16 * MB) {
+    const bf16* x[MB];
+#pragma unroll
+    for (int j = 0; j < MB; ++j) {
+      const int r = r_lo + min(c0 + 16 * j + ri, cnt - 1);
+      x[j] = A + (size_t)(a_rows ? a_rows[r] : r) * K + 8 * g;
+    }
+    f32x4 acc[RT][MB];
+#pragma unroll
+    for (int i = 0; i < RT; ++i)
+#pragma unroll
+      for (int j = 0; j < MB; ++j) acc[i][j] = f32x4{0.f, 0.f, 0.f, 0.f};
+    constexpr int U = RT * MB == 1 ? 8 : 4;  // steps in flight; the last group repeats its last step with zero tokens
+    for (int s = s0; s < s1; s += U) {
+      bf16x8 wf[U][RT], xf[U][MB];
+#pragma unroll
+      for (int q = 0; q < U; ++q) {
+        const int sc = min(s + q, s1 - 1);
+#pragma unroll
+        for (int i = 0; i < RT; ++i) wf[q][i] = load8(w + (size_t)16 * i * K + 32 * sc);
+#pragma unroll
+        for (int j = 0; j < MB; ++j) xf[q][j] = load8(x[j] + 32 * sc);
+      }
+#pragma unroll
+      for (int q = 0; q < U; ++q) {
+        const bool in = s + q < s1;
+#pragma unroll
+        for (int j = 0; j < MB; ++j) {
+#pragma unroll
+          for (int z = 0; z < 8; ++z) xf[q][j][z] = in ? xf[q][j][z] : (bf16)0.f;
+#pragma unroll
+          for (int i = 0; i < RT; ++i) acc[i][j] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(wf[q][i], xf[q][j], acc[i][j], 0, 0, 0);
+        }
+      }
+    }
+    __syncthreads();  // the previous round's sums are consumed
+#pragma unroll
+    for (int i = 0; i < RT; ++i)
+#pragma unroll
+      for (int j = 0; j < MB; ++j)
+        *reinterpret_cast<f32x4*>(&red[wv][i * MB + j][4 * lane]) = acc[i][j];
+    __syncthreads();
+    // element x of a tile: lane x / 4 (channel 4 (lane / 16) + x % 4, token lane % 16)
+    constexpr int NO = (ACT == 1 || ACT == 3) ? RT / 2 : RT;  // output tiles of 16 channels
+    const int No = (ACT == 1 || ACT == 3) ? N / 2 : N;
+    for (int o = tid; o < NO * MB * 256; o += 512) {
+      const int y = o & 255, j = (o >> 8) % MB, i = (o >> 8) / MB;
+      const int tok = c0 + 16 * j + ((y >> 2) & 15), ch = 4 * (y >> 6) + (y & 3);
+      if (tok >= cnt) continue;
+      float v = 0.f, u = 0.f;
+#pragma unroll
+      for (int q = 0; q < 8; ++q) {
+        v += red[q][((ACT == 1 || ACT == 3) ? 2 * i : i) * MB + j][y];
+        if (ACT == 1 || ACT == 3) u += red[q][(2 * i + 1) * MB + j][y];
+      }
+      if (ACT == 1 || ACT == 3) v = glu_pair<ACT>(v, u, actp);
+      if (ACT == 2) v = fmaxf(v, 0.f) * fmaxf(v, 0.f);
+      C[(size_t)(r_lo + tok) * No + (n0 / (RT / NO)) + 16 * i + ch] = (bf16)v;
+    }
+  }
+}
+
+static bool moe_gemm_stream(const void* A, const int* a_rows, const void* W, void* C, const int* offs, int E, int rows_total,
+                            int N, int K, int act, hipStream_t st, float actp) {
+  const bool glu = act == 1 || act == 3;
+  // gated products of more rows are bound by their weight bytes on the 128-row tiles already
+  if (K % 32 || N % 32 || rows_total > (glu ? 64 : 256) || rows_total > 32 * E) return false;
+#define GAI_MS(ACT_, RT_, MB_)                                                                                      \
+  moe_gemm_stream_kernel<ACT_, RT_, MB_><<<dim3(N / (16 * RT_), E), 512, 0, st>>>((const bf16*)A, a_rows, (const bf16*)W, \
+                                                                                  (bf16*)C, offs, N, K, actp)
+  const bool few = rows_total <= 16;
+  switch (act) {
+    case 0: if (few) GAI_MS(0, 1, 1); else GAI_MS(0, 2, 2); break;
+    case 1: if (few) GAI_MS(1, 2, 1); else GAI_MS(1, 2, 2); break;
+    case 2: if (few) GAI_MS(2, 1, 1); else GAI_MS(2, 2, 2); break;
+    default: if (few) GAI_MS(3, 2, 1); else GAI_MS(3, 2, 2); break;
+  }
+#undef GAI_MS
+  GAI_LAUNCH_CHECK();
+  return true;
+}
+
 void gai_moe_gemm(const void* A, const int* a_rows, const void* W, void* C, const int* offs, int E, int rows_total,
                   int N, int K, int act, hipStream_t st, int dt, float actp) {
   if (rows_total == 0) return;
@@ -658,6 +755,7 @@ void gai_moe_gemm(const void* A, const int* a_rows, const void* W, void* C, cons
   }
   // decode steps (<= 64 expert rows in all): every expert's weights streamed once by the decode kernel
   if (gai_moe_gemm_dec2(A, a_rows, W, C, offs, E, rows_total, N, K, act, st, actp)) return;
+  if (moe_gemm_stream(A, a_rows, W, C, offs, E, rows_total, N, K, act, st, actp)) return;
   const dim3 grid((rows_total + MBM - 1) / MBM + E, (N + MBN - 1) / MBN);
   const int lds = 4 * kMTile;
   static bool once = false;

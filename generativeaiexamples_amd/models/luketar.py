@@ -266,9 +266,15 @@ class LuketarModel(HybridDecoderBase):
             if ml is None:
                 continue
             q = p + "mlp."
-            gate_up = lambda n: mat(pad16(torch.cat([sd[n + "gate"].float(), sd[n + "up"].float()])))  # noqa: E731
+            def plain_ff(src, dst):
+                # wide feed-forwards padded with zeros to the split-K decode GEMM's grid (a zero gate row contributes nothing)
+                F_ = sd[src + "gate"].shape[0]
+                z = torch.zeros((-F_) % 512 if dt == torch.bfloat16 and F_ >= 1024 else 0, D)
+                w[dst + "in"] = mat(pad16(torch.cat([sd[src + "gate"].float(), z, sd[src + "up"].float(), z])))
+                w[dst + "down"] = mat(torch.cat([sd[src + "down"].float(), z.t()], 1))
+
             if ml["kind"] == "dense":
-                w[q + "in"], w[q + "down"] = gate_up(q), mat(sd[q + "down"])
+                plain_ff(q, q)
                 continue
             E, F_ = ml["router"]["experts"], ml["expert"]["ff"]
             # router rows padded to the GEMM's 16-column grid: the logits come out of the MFMA kernel in fp32
@@ -280,7 +286,7 @@ class LuketarModel(HybridDecoderBase):
             w[q + "e.down"] = mat(torch.stack([torch.cat([sd[q + f"e{e}.down"].float(), torch.zeros(D, Fp - F_)], 1)
                                                for e in range(E)]))
             if ml.get("shared"):
-                w[q + "shared.in"], w[q + "shared.down"] = gate_up(q + "shared."), mat(sd[q + "shared.down"])
+                plain_ff(q + "shared.", q + "shared.")
         self._alloc_state()
         return self
 

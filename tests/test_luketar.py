@@ -453,6 +453,25 @@ def test_latent_attention_bf16_against_reference(R, H):
 
 
 @_GPU
+@pytest.mark.parametrize("act", [None, "relu2", "swiglu", "clamp_glu"])
+@pytest.mark.parametrize("T,E,k,N,K", [(1, 8, 2, 96, 192), (7, 4, 2, 64, 320), (30, 6, 2, 160, 64), (60, 8, 3, 32, 1408)])
+def test_decode_sized_expert_products(T, E, k, N, K, act):
+    """Grouped expert products of a few rows whose K is off the staged weight stream's grid: some experts without rows, one
+    with most of them, every activation, against fp32 products of the same bf16 values."""
+    g = torch.Generator().manual_seed(2)
+    rn = lambda *s: torch.randn(*s, generator=g)  # noqa: E731
+    x, W = rn(T, K).to(torch.bfloat16), (rn(E, N, K) * K ** -0.5).to(torch.bfloat16)
+    ids = torch.stack([torch.randperm(E - 1, generator=g)[:k] for _ in range(T)]).int()     # the last expert gets none
+    ids[:, 0] = torch.where(torch.rand(T, generator=g) < 0.7, torch.zeros(T), ids[:, 0].float()).int()
+    rows, offs, _ = ops.moe_dispatch(ids.cuda(), E)
+    for gather in (True, False):
+        a = x if gather else x[rows.cpu().long()]
+        got = ops.moe_gemm(a.cuda(), rows if gather else None, W.cuda(), offs, T * k, act=act, act_param=0.7).float().cpu()
+        want = ops.moe_gemm(a.float(), rows.cpu() if gather else None, W.float(), offs.cpu(), T * k, act=act, act_param=0.7)
+        assert (got - want).norm() < 6e-3 * want.norm() and (got - want).abs().max() < 0.05 * want.abs().max()
+
+
+@_GPU
 def test_matrix_core_kernels_in_model():
     """bf16 model with sizes on the matrix-core grids: portions take the matrix-core kernels, single tokens the
     decode kernels; both against the oracle, alone and in a mixed batch."""
