@@ -1237,7 +1237,7 @@ def sigmoid_attention(q, k_cache, v_cache, block_tables, cu_q, ctx, H: int, G: i
     ns = native().sigmoid_attention_splits(T, S, H)
     part = torch.empty(ns * T * H * DV, dtype=torch.float32, device=q.device) if ns > 1 else None
     native().window_attention(q, k_cache, v_cache, block_tables, cu_q, ctx, out, H, G, DK, DV, float(scale), 0.0,
-                              int(window or 0), None, None, None, bias, True, float(out_scale), part, 0, None, None)
+                              int(window or 0), None, None, None, bias, True, float(out_scale), part, 0, None, None, None)
     return out
 
 
