@@ -38,7 +38,7 @@ from .. import ops
 from ..engine.state_pool import StatePool
 from ..parallel.dist import DistContext, get_context
 from .common import ForwardBatch
-from .hybrid_base import HybridDecoderBase
+from .hybrid_base import HybridDecoderBase, stack_gated_experts
 
 MIXERS = ("latent_attention", "mlstm")
 DEN_EPS = 1e-6         # added to the matrix memory's denominator
@@ -276,15 +276,11 @@ class LuketarModel(HybridDecoderBase):
             if ml["kind"] == "dense":
                 plain_ff(q, q)
                 continue
-            E, F_ = ml["router"]["experts"], ml["expert"]["ff"]
+            E = ml["router"]["experts"]
             # router rows padded to the GEMM's 16-column grid: the logits come out of the MFMA kernel in fp32
             w[q + "router"], w[q + "router.b"] = mat(pad16(sd[q + "router"])), f32(sd[q + "router.b"])
-            Fp = F_ + (-F_) % (64 if dt == torch.bfloat16 else 16)
-            zr = lambda t: torch.cat([t.float(), torch.zeros(Fp - F_, D)])  # noqa: E731
-            w[q + "gate_up"] = mat(torch.stack([ops.interleave_gate_up(zr(sd[q + f"e{e}.gate"]), zr(sd[q + f"e{e}.up"]))
-                                                for e in range(E)]))
-            w[q + "e.down"] = mat(torch.stack([torch.cat([sd[q + f"e{e}.down"].float(), torch.zeros(D, Fp - F_)], 1)
-                                               for e in range(E)]))
+            gate_up, down = stack_gated_experts(sd, q, E, 64 if dt == torch.bfloat16 else 16)
+            w[q + "gate_up"], w[q + "e.down"] = mat(gate_up), mat(down)
             if ml.get("shared"):
                 plain_ff(q + "shared.", q + "shared.")
         self._alloc_state()

@@ -42,7 +42,7 @@ from .. import ops
 from ..engine.state_pool import StatePool
 from ..parallel.dist import DistContext, get_context
 from .common import ForwardBatch
-from .hybrid_base import HybridDecoderBase
+from .hybrid_base import HybridDecoderBase, loop_runs
 
 MIXERS = ("attention", "wkv", "channel_delta")
 
@@ -93,13 +93,7 @@ class PinavikConfig:
 
     def runs(self) -> List[Tuple[int, int]]:
         """Execution order as (layer, pass) pairs; a looped layer appears once per pass."""
-        n = len(self.layers)
-        if not self.loop_times:
-            return [(i, 0) for i in range(n)]
-        out = [(i, 0) for i in range(self.loop_start)]
-        for t in range(self.loop_times):
-            out += [(i, t) for i in range(self.loop_start, self.loop_stop)]
-        return out + [(i, 0) for i in range(self.loop_stop, n)]
+        return loop_runs(len(self.layers), self.loop_start, self.loop_stop, self.loop_times)
 
     @staticmethod
     def from_json(path_or_dict) -> "PinavikConfig":

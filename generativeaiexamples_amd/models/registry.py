@@ -8,6 +8,7 @@ from typing import Optional, Tuple
 import torch
 
 from ..engine.tokenizer import Tokenizer, bert_byte_tokenizer, load_tokenizer, llama3_byte_tokenizer, small_byte_tokenizer
+from .bamanex import BamanexConfig, BamanexModel
 from .bert import BertConfig, BertModel
 from .clip import ClipConfig, ClipModel
 from .decoder_reranker import DecoderRerankerConfig, DecoderRerankerModel
@@ -58,6 +59,10 @@ LLM_PRESETS = {
     # routed clamped gated experts plus a shared expert)
     "tiny-luketar": ("tiny-luketar", lambda: LuketarConfig.tiny()),
     "luketar-1b": ("luketar-1b", lambda: LuketarConfig.sized(2048, 12, 5632, 16, 128)),
+    # windowed attention beside the feed-forward (parallel layers), unit-norm rotated queries / keys, sinks, head gates,
+    # dense and routed layers, a looped block
+    "tiny-bamanex": ("tiny-bamanex", lambda: BamanexConfig.tiny()),
+    "bamanex-1b": ("bamanex-1b", lambda: BamanexConfig.sized(2048, 12, 5632, 16, 128)),
     "opt-125m": ("facebook/opt-125m", lambda: OPTConfig.opt_125m()),
     "mixtral-8x7b": ("mistralai/mixtral-8x7b-instruct-v0.1", lambda: MixtralConfig.mixtral_8x7b()),
     "tiny-moe": ("tiny-moe", lambda: MixtralConfig.tiny_moe()),
@@ -105,6 +110,8 @@ def build_llm(preset: str = "llama3-8b", weights: Optional[str] = None, device=N
             m = VipolixModel(VipolixConfig.from_json(weights), device=device, dtype=dtype or torch.bfloat16)
         elif arch == "luketar":
             m = LuketarModel(LuketarConfig.from_json(weights), device=device, dtype=dtype or torch.bfloat16)
+        elif arch == "bamanex":
+            m = BamanexModel(BamanexConfig.from_json(weights), device=device, dtype=dtype or torch.bfloat16)
         elif arch == "opt":
             m = OPTModel(OPTConfig.from_hf(weights), device=device)
         elif arch == "mixtral":
@@ -150,6 +157,9 @@ def build_llm(preset: str = "llama3-8b", weights: Optional[str] = None, device=N
         vocab = cfg.vocab_size
     elif isinstance(cfg, LuketarConfig):
         m = LuketarModel(cfg, device=device, dtype=dtype or torch.bfloat16).random_init(seed)
+        vocab = cfg.vocab_size
+    elif isinstance(cfg, BamanexConfig):
+        m = BamanexModel(cfg, device=device, dtype=dtype or torch.bfloat16).random_init(seed)
         vocab = cfg.vocab_size
     else:
         m = LlamaModel(cfg, device=device).random_init(seed)

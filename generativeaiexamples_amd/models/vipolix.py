@@ -46,7 +46,7 @@ from .. import ops
 from ..engine.state_pool import StatePool
 from ..parallel.dist import DistContext, get_context
 from .common import ForwardBatch
-from .hybrid_base import HybridDecoderBase
+from .hybrid_base import HybridDecoderBase, stack_gated_experts
 
 MIXERS = ("gla", "parallel")
 ROUTE_EPS = 1e-20               # added to the sum of the chosen router scores
@@ -305,17 +305,13 @@ class VipolixModel(HybridDecoderBase):
             if ml is not None:
                 w[p + "norm2"] = f32(1 + sd[p + "norm2"].float())
                 q = p + "mlp."
-                E, F_ = ml["router"]["experts"], ml["expert"]["ff"]
+                E = ml["router"]["experts"]
                 # router rows padded to the GEMM's 16-column grid: the logits come out of the MFMA kernel in fp32
                 w[q + "router"] = mat(pad16(sd[q + "router"]))
                 if (q + "correction") in sd:
                     w[q + "correction"] = f32(sd[q + "correction"])
-                Fp = F_ + (-F_) % (64 if dt == torch.bfloat16 else 16)
-                zr = lambda t: torch.cat([t.float(), torch.zeros(Fp - F_, D)])  # noqa: E731
-                w[q + "gate_up"] = mat(torch.stack([ops.interleave_gate_up(zr(sd[q + f"e{e}.gate"]), zr(sd[q + f"e{e}.up"]))
-                                                    for e in range(E)]))
-                w[q + "down"] = mat(torch.stack([torch.cat([sd[q + f"e{e}.down"].float(), torch.zeros(D, Fp - F_)], 1)
-                                                 for e in range(E)]))
+                gate_up, down = stack_gated_experts(sd, q, E, 64 if dt == torch.bfloat16 else 16)
+                w[q + "gate_up"], w[q + "down"] = mat(gate_up), mat(down)
                 if ml.get("shared"):
                     rows = [sd[q + "shared.gate"].float(), sd[q + "shared.up"].float()]
                     if (q + "shared.sg") in sd:

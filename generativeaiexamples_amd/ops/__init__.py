@@ -15,7 +15,7 @@ import numpy as np
 import torch
 
 from . import reference as ref
-from .reference import BLOCK, interleave_gate_up, rope_cos_sin  # noqa: F401
+from .reference import BLOCK, interleave_gate_up, rope_cos_sin, rope_inv_freq  # noqa: F401
 
 _C = None
 _C_ERR: Exception | None = None
@@ -864,11 +864,12 @@ def moe_route(logits: torch.Tensor, k: int, renorm: bool = True, score: str = "s
     if not logits.is_cuda:
         if bias is not None:
             return ref.moe_route_biased(logits, k, bias, eps)
-        return ref.moe_route_sigmoid(logits, k) if score == "sigmoid" else ref.moe_route(logits, k, renorm)
+        return ref.moe_route_sigmoid(logits, k) if score == "sigmoid" else ref.moe_route(logits, k, renorm, eps)
     T = logits.shape[0]
     ids = torch.empty(T, k, dtype=torch.int32, device=logits.device)
     w = torch.empty(T, k, dtype=torch.float32, device=logits.device)
-    native().moe_route(logits.float().contiguous(), k, renorm, ids, w, score == "sigmoid", bias, float(eps))
+    x = logits.float()
+    native().moe_route(x if x.stride(1) == 1 else x.contiguous(), k, renorm, ids, w, score == "sigmoid", bias, float(eps))
     return ids, w
 
 
@@ -1190,25 +1191,28 @@ def window_attention(q, k_cache, v_cache, block_tables, cu_q, ctx, H: int, G: in
     own chunk of positions, floor(j / chunk) == floor(i / chunk) (chunk > 0), or all. Scores are capped by softcap *
     tanh(s / softcap) and lowered by r1_h ln(1 + r2_h distance); head_scale (fp32 [H]) multiplies the scores of a head;
     sink (a score, or an fp32 [H] tensor of scores, one per head) adds exp(sink) to the softmax denominator without a
-    value (sink = 0: one is added). Output [T, H * DV] times out_scale, times sigmoid(gate) when given (`out` may be a column slice of a wider buffer)."""
+    value (sink = 0: one is added). Output [T, H * DV] times out_scale, times sigmoid(gate) when given: gate [T, H * DV]
+    (an element at a time) or [T, H] (one number per head), both column slices of a wider projection (`out` may be a
+    column slice of a wider buffer)."""
     if not q.is_cuda:
         if chunk or head_scale is not None or sink is not None or out_scale != 1.0:
-            if softcap or r1 is not None or gate is not None:
-                raise ValueError("window_attention: chunks, head scales and sinks go without cap, distance term and gate")
+            if softcap or r1 is not None:
+                raise ValueError("window_attention: chunks, head scales and sinks go without cap and distance term")
             return _into(out, ref.masked_attention(q, k_cache, v_cache, block_tables, cu_q, ctx, H, G, DK, DV, scale,
-                                                   int(window or 0), int(chunk or 0), head_scale, sink, out_scale))
+                                                   int(window or 0), int(chunk or 0), head_scale, sink, out_scale, gate))
         return _into(out, ref.window_attention(q, k_cache, v_cache, block_tables, cu_q, ctx, H, G, DK, DV, scale,
                                                softcap, window, r1, r2, gate))
     if out is None:
         out = torch.empty(q.shape[0], H * DV, dtype=q.dtype, device=q.device)
     hs = sink if isinstance(sink, torch.Tensor) else None
-    if (G == 1 and q.dtype == torch.bfloat16 and not softcap and r1 is None and gate is None and not chunk
+    if (q.dtype == torch.bfloat16 and not softcap and r1 is None and (gate is None or gate.shape[1] == H) and not chunk
             and head_scale is None and out_scale == 1.0 and (sink is None or hs is not None)
-            and native().mqa_attention_ok(DK, DV)):
-        # one kv head: (token, head) rows share the keys, so tiles mix heads and tokens (attention_mqa.hip)
-        n = native().mqa_attention_ws_floats(q.shape[0], ctx.numel(), H, DV)
+            and native().gqa_attention_ok(DK, DV)):
+        # (token, head) rows of one kv head share the keys, so tiles mix heads and tokens (attention_gqa.hip)
+        n = native().gqa_attention_ws_floats(q.shape[0], ctx.numel(), H, G, DV)
         ws = torch.empty(n, dtype=torch.float32, device=q.device) if n else None
-        native().mqa_attention(q, k_cache, v_cache, block_tables, cu_q, ctx, out, H, float(scale), int(window or 0), hs, ws)
+        native().gqa_attention(q, k_cache, v_cache, block_tables, cu_q, ctx, out, H, G, float(scale), int(window or 0), hs,
+                               gate, ws)
         return out
     # decode steps of few rows: the keys of a row are split over several waves, merged from (sums, maximum, denominator)
     T, S = q.shape[0], ctx.numel()
@@ -1559,3 +1563,34 @@ def mlstm(q, k, v, ig, fg, ib, fb, cap: float, gate, norm_w, S, n, m, cu, slots,
     native().mlstm(q, k, v, ig, fg, ib, fb, float(cap), gate, norm_w, S, n, m, cu, slots, float(q_scale), float(eps),
                    float(den_eps), y, ws)
     return y
+
+
+# ---------------------------------------------------------------------------------------------
+# parallel (mixer beside feed-forward) residual, rotate-half positions with unit-norm queries and keys
+# ---------------------------------------------------------------------------------------------
+def parallel_add_norm_f32(res, a=None, sa=None, b=None, sb=None, w1=None, w2=None, eps: float = 1e-6, out_dtype=None):
+    """The pass between two parallel layers: fp32 ``res`` (in place) += sa * a + sb * b - the two branch outputs times
+    their per-channel scales (fp32 [D]; None: one) - and the next layer's two norms of the new sum, rmsnorm(res) * w1 and
+    rmsnorm(res) * w2 in out_dtype (None where no weight is given). One read of the stream, one set of statistics."""
+    if not res.is_cuda:
+        return ref.parallel_add_norm_f32(res, a, sa, b, sb, w1, w2, eps, out_dtype)
+    h1, h2 = (torch.empty(res.shape, dtype=out_dtype, device=res.device) if w is not None else None for w in (w1, w2))
+    native().parallel_add_norm_f32(res, a, sa, b, sb, w1, h1, w2, h2, float(eps))
+    return h1, h2
+
+
+def rotary_half_kv_write(q, k, v, positions, slots, k_cache, v_cache, H: int, G: int, DK: int, DV: int, inv_freq,
+                         unit_eps: Optional[float] = None):
+    """Rotation in the rotate-half layout: the channel pairs (i, i + n), i < n = len(inv_freq), of every q and k head
+    turned by position * inv_freq[i] (inv_freq: fp64 [n], see rope_inv_freq; angles formed and reduced in fp64; channels
+    past 2 n pass unchanged); with unit_eps, every q and k head is then divided by its root mean square (eps inside the
+    root, no weight). k and v go into their cache slots; returns q [T, H * DK]. q / k / v may be column slices of one
+    projection."""
+    if 2 * inv_freq.numel() > DK:
+        raise ValueError("rotary_half_kv_write: more rotated channels than a head has")
+    if not q.is_cuda:
+        return ref.rotary_half_kv_write(q, k, v, positions, slots, k_cache, v_cache, H, G, DK, DV, inv_freq, unit_eps)
+    q_out = torch.empty(q.shape[0], H * DK, dtype=k_cache.dtype, device=q.device)
+    native().rotary_half_kv_write(q, k, v, positions, slots, q_out, k_cache, v_cache, H, G, DK, DV, inv_freq,
+                                  -1.0 if unit_eps is None else float(unit_eps))
+    return q_out

@@ -71,6 +71,23 @@ def interleave_gate_up(gate: torch.Tensor, up: torch.Tensor) -> torch.Tensor:
     return torch.stack([gate.reshape(I // 16, 16, K), up.reshape(I // 16, 16, K)], 1).reshape(2 * I, K)
 
 
+def rope_inv_freq(dims: int, base: float, scaling: dict | None = None) -> torch.Tensor:
+    """fp64 [dims / 2] angle steps per position base^(-2i / dims). ``scaling`` {"factor", "low", "high", "original"}:
+    frequency-dependent (Llama-3.1) scaling - wavelengths shorter than original / high are kept, those longer than
+    original / low are stretched by factor, a linear ramp in turns per `original` positions between the two."""
+    inv = 1.0 / (float(base) ** (torch.arange(0, dims, 2, dtype=torch.float64) / max(dims, 1)))
+    if scaling:
+        factor, old = float(scaling["factor"]), float(scaling["original"])
+        lf, hf = float(scaling["low"]), float(scaling["high"])
+        low_wl, high_wl = old / lf, old / hf
+        wl = 2 * math.pi / inv
+        smooth = (old / wl - lf) / (hf - lf)
+        scaled = torch.where(wl > low_wl, inv / factor, inv)
+        mid = (wl <= low_wl) & (wl >= high_wl)
+        inv = torch.where(mid, (1 - smooth) * inv / factor + smooth * inv, scaled)
+    return inv
+
+
 def rope_cos_sin(max_pos: int, head_dim: int, theta: float = 500000.0, scaling: dict | None = None,
                  device=None) -> torch.Tensor:
     """fp32 table [max_pos, D] = [cos(D/2) | sin(D/2)], neox rotate-half convention.
@@ -78,17 +95,11 @@ def rope_cos_sin(max_pos: int, head_dim: int, theta: float = 500000.0, scaling: 
     ``scaling`` implements the Llama-3.1 frequency-dependent rope scaling
     ({"factor", "low_freq_factor", "high_freq_factor", "original_max_position_embeddings"}).
     """
-    inv = 1.0 / (theta ** (torch.arange(0, head_dim, 2, dtype=torch.float64) / head_dim))
     if scaling:
-        factor = scaling.get("factor", 8.0)
-        lf, hf = scaling.get("low_freq_factor", 1.0), scaling.get("high_freq_factor", 4.0)
-        old = scaling.get("original_max_position_embeddings", 8192)
-        low_wl, high_wl = old / lf, old / hf
-        wl = 2 * math.pi / inv
-        smooth = (old / wl - lf) / (hf - lf)
-        scaled = torch.where(wl > low_wl, inv / factor, inv)
-        mid = (wl <= low_wl) & (wl >= high_wl)
-        inv = torch.where(mid, (1 - smooth) * inv / factor + smooth * inv, scaled)
+        scaling = dict(factor=scaling.get("factor", 8.0), low=scaling.get("low_freq_factor", 1.0),
+                       high=scaling.get("high_freq_factor", 4.0),
+                       original=scaling.get("original_max_position_embeddings", 8192))
+    inv = rope_inv_freq(head_dim, theta, scaling)
     t = torch.arange(max_pos, dtype=torch.float64)
     f = torch.outer(t, inv)
     return torch.cat([f.cos(), f.sin()], -1).float().to(device)
@@ -252,11 +263,11 @@ def sim_topk(Q, X, bias, n_rows, k):
     return v, i
 
 
-def moe_route(logits, k, renorm=True):
+def moe_route(logits, k, renorm=True, eps=0.0):
     p = logits.float().softmax(-1)
     w, ids = torch.topk(p, k, dim=-1)
     if renorm:
-        w = w / w.sum(-1, keepdim=True)
+        w = w / (w.sum(-1, keepdim=True) + eps)
     return ids.int(), w
 
 
@@ -519,10 +530,9 @@ def window_attention(q, k_cache, v_cache, block_tables, cu_q, ctx, H, G, DK, DV,
                 sc = sc - float(r1[h]) * torch.log1p(float(r2[h]) * dist.clamp(min=0).float())
             sc = sc.masked_fill(~vis, float("-inf"))
             out[b:e, h] = torch.softmax(sc, -1) @ V[h // (H // G)]
-    out = out.reshape(T, H * DV)
     if gate is not None:
-        out = out * torch.sigmoid(gate.float())
-    return out.to(q.dtype)
+        out = out * torch.sigmoid(gate.float().reshape(T, H, -1))
+    return out.reshape(T, H * DV).to(q.dtype)
 
 
 def token_shift_mix(h, mu, shift_state, cu, slots):
@@ -925,10 +935,11 @@ def rotary_kv_write(q, k, v, positions, slots, k_cache, v_cache, H, G, DK, DV, r
 
 
 def masked_attention(q, k_cache, v_cache, block_tables, cu_q, ctx, H, G, DK, DV, scale, window, chunk, head_scale, sink,
-                     out_scale):
+                     out_scale, gate=None):
     """Softmax attention over the visible keys j <= i: the last `window` ones (window > 0), those of the query's own
     chunk of positions floor(i / chunk) = floor(j / chunk) (chunk > 0), or all. head_scale [H] multiplies the scores of
-    a head; sink (a score, fp32 [H] scores, or None) adds exp(sink) to the softmax denominator without adding a value."""
+    a head; sink (a score, fp32 [H] scores, or None) adds exp(sink) to the softmax denominator without adding a value;
+    gate: the output times its sigmoid, an element [T, H * DV] or a head [T, H] at a time."""
     T = q.numel() // (H * DK)
     q3 = q.float().view(T, H, DK)
     out = torch.zeros(T, H, DV)
@@ -961,6 +972,8 @@ def masked_attention(q, k_cache, v_cache, block_tables, cu_q, ctx, H, G, DK, DV,
             if sk is not None:
                 den = den + torch.exp(float(sk) - m)
             out[b:e, h] = (p / den) @ V[h // (H // G)]
+    if gate is not None:
+        out = out * torch.sigmoid(gate.float().reshape(T, H, -1))
     return (out.reshape(T, H * DV) * float(out_scale)).to(q.dtype)
 
 
@@ -1117,3 +1130,35 @@ def moe_route_chosen(logits, k, bias):
     z = logits.float() + bias.float() if bias is not None else logits.float()
     v, ids = torch.topk(z, k, dim=-1)
     return ids.int(), torch.softmax(v, -1)
+
+
+# ---------------------------------------------------------------------------------------------
+# parallel (mixer beside feed-forward) residual, rotate-half positions with unit-norm queries and keys
+# ---------------------------------------------------------------------------------------------
+def parallel_add_norm_f32(res, a, sa, b, sb, w1, w2, eps, out_dtype):
+    """res (fp32, in place) += sa * a (+ sb * b); -> (rmsnorm(res) * w1, rmsnorm(res) * w2) as out_dtype, None without
+    their weight."""
+    for y, s in ((a, sa), (b, sb)):
+        if y is not None:
+            res.add_(y.float() * s.float() if s is not None else y.float())
+    n = res * torch.rsqrt(res.pow(2).mean(-1, keepdim=True) + eps)
+    return tuple((n * w.float()).to(out_dtype) if w is not None else None for w in (w1, w2))
+
+
+def rotary_half_kv_write(q, k, v, positions, slots, k_cache, v_cache, H, G, DK, DV, inv_freq, unit_eps):
+    """Channels (i, i + n) of every q and k head turned by position * inv_freq[i], i < n = len(inv_freq) (the rest
+    unchanged), then divided by the head's root mean square (unit_eps given); k and v into their cache slots; returns q."""
+    T, n = q.shape[0], inv_freq.numel()
+    ang = positions[:T].to(torch.float64)[:, None] * inv_freq.to(torch.float64)
+    c, s = torch.cos(ang).float()[:, None, :], torch.sin(ang).float()[:, None, :]
+
+    def turn(x):
+        x = x.float()
+        u, w = x[..., :n], x[..., n:2 * n]
+        x = torch.cat([u * c - w * s, w * c + u * s, x[..., 2 * n:]], -1)
+        return x if unit_eps is None else x * torch.rsqrt(x.pow(2).mean(-1, keepdim=True) + unit_eps)
+
+    sl = slots[:T].long()
+    k_cache[sl // BLOCK, :, sl % BLOCK] = turn(k.reshape(T, G, DK)).to(k_cache.dtype)
+    v_cache[sl // BLOCK, :, :, sl % BLOCK] = v.reshape(T, G, DV).to(v_cache.dtype)
+    return turn(q.reshape(T, H, DK)).reshape(T, H * DK).to(k_cache.dtype)
