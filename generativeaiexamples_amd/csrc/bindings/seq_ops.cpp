@@ -1,5 +1,5 @@
 // PyTorch bindings of the sequence-mixer kernels with a 32-bit residual / state (norm_f32.hip, attention_window.hip,
-// recurrent.hip, hyper.hip, head_linear.hip, mlstm.hip). Shape / dtype checks on the host, a launch on the current stream, no allocation: graph-capturable.
+// attention_gqa.hip, recurrent.hip, hyper.hip, head_linear.hip, mlstm.hip). Shape / dtype checks on the host, a launch on the current stream, no allocation: graph-capturable.
 // Activation tensors are bf16 or fp32 (all of one call alike); per-channel tables and states are fp32.
 #include <torch/extension.h>
 #include <c10/hip/HIPStream.h>
@@ -200,11 +200,12 @@ void window_attention(const Tensor& q, const Tensor& k_cache, const Tensor& v_ca
   if (sigmoid) TORCH_CHECK(!gate && !r1 && softcap == 0.0, "window_attention: sigmoid mode takes no cap, distance term or gate");
   TORCH_CHECK(r1.has_value() == r2.has_value(), "window_attention: r1 and r2 come together");
   if (r1) TORCH_CHECK(r1->numel() == H && r2->numel() == H, "window_attention: one distance pair per head");
-  int ldg = 0;
-  if (gate) {  // output multiplied by sigmoid(gate), [T, H * DV] rows of a wider projection
+  int ldg = 0, ghead = 0;
+  if (gate) {  // output multiplied by sigmoid(gate), [T, H * DV] or [T, H] rows of a wider projection
     same_dt(*gate, dt, "gate");
     ldg = row_stride(*gate, "gate");
-    TORCH_CHECK(gate->size(0) == T && gate->size(1) == H * DV, "window_attention: gate shape");
+    TORCH_CHECK(gate->size(0) == T && (gate->size(1) == H * DV || gate->size(1) == H), "window_attention: gate shape");
+    ghead = gate->size(1) == H ? 1 : 0;
   }
   float* partp = nullptr;
   if (part) {  // scratch of the key-split decode form (softmax mode keeps a maximum and a denominator per row too)
@@ -219,7 +220,7 @@ void window_attention(const Tensor& q, const Tensor& k_cache, const Tensor& v_ca
                        r2 ? f32(*r2, "r2") : nullptr, gate ? gate->data_ptr() : nullptr, ldg,
                        sig_bias ? f32(*sig_bias, "sig_bias") : nullptr, sigmoid ? 1 : 0, (float)out_scale, dt,
                        cur_stream(), partp, (int)chunk, head_scale ? f32(*head_scale, "head_scale") : nullptr, sink ? 1 : 0,
-                       sink ? (float)*sink : 0.f, head_sink ? f32(*head_sink, "head_sink") : nullptr);
+                       sink ? (float)*sink : 0.f, head_sink ? f32(*head_sink, "head_sink") : nullptr, ghead);
 }
 
 void rotary_kv_write(const Tensor& q, const Tensor& k, const Tensor& v, const Tensor& positions, const Tensor& slots,
@@ -557,31 +558,88 @@ void selective_scan(const Tensor& x, const Tensor& dt, const Tensor& dt_bias, co
                      I, N, dtt, cur_stream());
 }
 
-int64_t mqa_attention_ws_floats(int64_t T, int64_t S, int64_t H, int64_t DV) {
-  return (int64_t)gai_mqa_attention_ws_floats((int)T, (int)S, (int)H, (int)DV);
+int64_t gqa_attention_ws_floats(int64_t T, int64_t S, int64_t H, int64_t G, int64_t DV) {
+  TORCH_CHECK(G >= 1 && H % G == 0, "gqa_attention: heads must be a multiple of kv heads");
+  return (int64_t)gai_gqa_attention_ws_floats((int)T, (int)S, (int)H, (int)G, (int)DV);
 }
 
-void mqa_attention(const Tensor& q, const Tensor& k_cache, const Tensor& v_cache, const Tensor& block_tables,
-                   const Tensor& cu_q, const Tensor& ctx, Tensor& out, int64_t H, double scale, int64_t window,
-                   const optional<Tensor>& sink, const optional<Tensor>& ws) {
-  TORCH_CHECK(act_dt(q, "q") == 0 && act_dt(out, "out") == 0, "mqa_attention: bf16");
+void gqa_attention(const Tensor& q, const Tensor& k_cache, const Tensor& v_cache, const Tensor& block_tables,
+                   const Tensor& cu_q, const Tensor& ctx, Tensor& out, int64_t H, int64_t G, double scale, int64_t window,
+                   const optional<Tensor>& sink, const optional<Tensor>& gate, const optional<Tensor>& ws) {
+  TORCH_CHECK(act_dt(q, "q") == 0 && act_dt(out, "out") == 0, "gqa_attention: bf16");
   const int DK = k_cache.size(3), DV = v_cache.size(2), S = ctx.numel();
-  check_cache(k_cache, v_cache, 0, 1, DK, DV);
-  TORCH_CHECK(gai_mqa_attention_ok(DK, DV), "mqa_attention: no kernel for these key / value sizes");
-  TORCH_CHECK(q.is_contiguous() && q.numel() % (H * DK) == 0, "mqa_attention: q shape");
+  check_cache(k_cache, v_cache, 0, G, DK, DV);
+  TORCH_CHECK(gai_gqa_attention_ok(DK, DV), "gqa_attention: no kernel for these key / value sizes");
+  TORCH_CHECK(q.is_contiguous() && q.numel() % (H * DK) == 0, "gqa_attention: q shape");
   const int T = q.numel() / (H * DK), ldo = row_stride(out, "out");
   TORCH_CHECK(out.size(0) == T && out.size(1) == H * DV && cu_q.numel() == S + 1 && block_tables.dim() == 2 &&
-                  block_tables.size(0) >= S, "mqa_attention: out / cu_q / block table shapes");
-  TORCH_CHECK(((size_t)out.data_ptr() & 7) == 0 && ldo % 4 == 0, "mqa_attention: output rows on a grid of four elements");
-  if (sink) TORCH_CHECK(sink->numel() == H, "mqa_attention: one sink score per head");
-  const int64_t need = mqa_attention_ws_floats(T, S, H, DV);
+                  block_tables.size(0) >= S, "gqa_attention: out / cu_q / block table shapes");
+  TORCH_CHECK(((size_t)out.data_ptr() & 7) == 0 && ldo % 4 == 0, "gqa_attention: output rows on a grid of four elements");
+  if (sink) TORCH_CHECK(sink->numel() == H, "gqa_attention: one sink score per head");
+  int ldg = 0;
+  if (gate) {
+    same_dt(*gate, 0, "gate");
+    ldg = row_stride(*gate, "gate");
+    TORCH_CHECK(gate->size(0) == T && gate->size(1) == H, "gqa_attention: one gate per token and head");
+  }
+  const int64_t need = gqa_attention_ws_floats(T, S, H, G, DV);
   if (need)
     TORCH_CHECK(ws && ws->is_cuda() && ws->scalar_type() == at::kFloat && ws->is_contiguous() && ws->numel() >= need,
-                "mqa_attention: workspace too small");
-  gai_mqa_attention(q.data_ptr(), k_cache.data_ptr(), v_cache.data_ptr(), i32(block_tables, "block_tables"),
-                    block_tables.size(1), i32(cu_q, "cu_q"), i32(ctx, "ctx"), S, out.data_ptr(), ldo, T, (int)H, DK, DV,
-                    (float)scale, (int)window, sink ? f32(*sink, "sink") : nullptr, need ? ws->data_ptr<float>() : nullptr,
-                    cur_stream());
+                "gqa_attention: workspace too small");
+  gai_gqa_attention(q.data_ptr(), k_cache.data_ptr(), v_cache.data_ptr(), i32(block_tables, "block_tables"),
+                    block_tables.size(1), i32(cu_q, "cu_q"), i32(ctx, "ctx"), S, out.data_ptr(), ldo, T, (int)H, (int)G, DK,
+                    DV, (float)scale, (int)window, sink ? f32(*sink, "sink") : nullptr, gate ? gate->data_ptr() : nullptr,
+                    ldg, need ? ws->data_ptr<float>() : nullptr, cur_stream());
+}
+
+void rotary_half_kv_write(const Tensor& q, const Tensor& k, const Tensor& v, const Tensor& positions, const Tensor& slots,
+                          Tensor& q_out, Tensor& k_cache, Tensor& v_cache, int64_t H, int64_t G, int64_t DK, int64_t DV,
+                          const Tensor& inv_freq, double unit_eps) {
+  const int dt = act_dt(q, "q");
+  same_dt(k, dt, "k");
+  same_dt(v, dt, "v");
+  same_dt(q_out, dt, "q_out");
+  check_cache(k_cache, v_cache, dt, G, DK, DV);
+  const int T = q.size(0);
+  TORCH_CHECK(q.size(1) == H * DK && k.size(0) == T && k.size(1) == G * DK && v.size(0) == T && v.size(1) == G * DV,
+              "rotary_half_kv_write: projection shapes");
+  TORCH_CHECK(slots.numel() >= T && positions.numel() >= T && q_out.is_contiguous() && q_out.numel() == (int64_t)T * H * DK,
+              "rotary_half_kv_write: slot / position / output shapes");
+  TORCH_CHECK(inv_freq.is_cuda() && inv_freq.scalar_type() == at::kDouble && inv_freq.is_contiguous() &&
+                  2 * inv_freq.numel() <= DK, "rotary_half_kv_write: fp64 frequencies of at most half a head's channels");
+  gai_rotary_half_kv_write(q.data_ptr(), row_stride(q, "q"), k.data_ptr(), row_stride(k, "k"), v.data_ptr(),
+                           row_stride(v, "v"), i32(positions, "positions"), i32(slots, "slots"), q_out.data_ptr(),
+                           k_cache.data_ptr(), v_cache.data_ptr(), T, H, G, DK, DV, inv_freq.data_ptr<double>(),
+                           (int)inv_freq.numel(), (float)unit_eps, dt, cur_stream());
+}
+
+void parallel_add_norm_f32(Tensor& res, const optional<Tensor>& a, const optional<Tensor>& sa, const optional<Tensor>& b,
+                           const optional<Tensor>& sb, const optional<Tensor>& w1, const optional<Tensor>& h1,
+                           const optional<Tensor>& w2, const optional<Tensor>& h2, double eps) {
+  float* r = f32w(res, "res");
+  TORCH_CHECK(res.dim() == 2, "parallel_add_norm_f32: res [T, D]");
+  const int T = res.size(0), D = res.size(1);
+  int dt = -1;
+  auto seen = [&](const optional<Tensor>& x, const char* name) {
+    if (!x) return;
+    const int d = act_dt(*x, name);
+    TORCH_CHECK(dt < 0 || dt == d, "parallel_add_norm_f32: branch outputs and normed rows share a dtype");
+    dt = d;
+    TORCH_CHECK(x->dim() == 2 && x->size(0) == T && x->size(1) == D, "parallel_add_norm_f32: ", name, " [T, D]");
+  };
+  seen(a, "a");
+  seen(b, "b");
+  seen(h1, "h1");
+  seen(h2, "h2");
+  TORCH_CHECK(dt >= 0, "parallel_add_norm_f32: nothing to do");
+  for (const auto* x : {&sa, &sb, &w1, &w2})
+    if (*x) TORCH_CHECK((*x)->numel() == D, "parallel_add_norm_f32: one scale / weight per channel");
+  TORCH_CHECK((!h1 || (w1 && h1->is_contiguous())) && (!h2 || (w2 && h2->is_contiguous())),
+              "parallel_add_norm_f32: contiguous outputs, each with a weight");
+  gai_parallel_add_norm_f32(r, a ? a->data_ptr() : nullptr, a ? row_stride(*a, "a") : 0, sa ? f32(*sa, "sa") : nullptr,
+                            b ? b->data_ptr() : nullptr, b ? row_stride(*b, "b") : 0, sb ? f32(*sb, "sb") : nullptr,
+                            w1 ? f32(*w1, "w1") : nullptr, h1 ? h1->data_ptr() : nullptr, w2 ? f32(*w2, "w2") : nullptr,
+                            h2 ? h2->data_ptr() : nullptr, T, D, (float)eps, dt, cur_stream());
 }
 
 void latent_norm_write(const Tensor& dq, const Tensor& wq, const Tensor& dkv, const Tensor& wkv, const Tensor& slots,
@@ -680,9 +738,11 @@ void mlstm(const Tensor& q, const Tensor& k, const Tensor& v, const Tensor& ig, 
 
 void gai_bind_seq_ops(pybind11::module_& m) {
   m.def("add_dyt_f32", &add_dyt_f32);
-  m.def("mqa_attention", &mqa_attention);
-  m.def("mqa_attention_ok", [](int64_t DK, int64_t DV) { return gai_mqa_attention_ok((int)DK, (int)DV) != 0; });
-  m.def("mqa_attention_ws_floats", &mqa_attention_ws_floats);
+  m.def("gqa_attention", &gqa_attention);
+  m.def("gqa_attention_ok", [](int64_t DK, int64_t DV) { return gai_gqa_attention_ok((int)DK, (int)DV) != 0; });
+  m.def("gqa_attention_ws_floats", &gqa_attention_ws_floats);
+  m.def("rotary_half_kv_write", &rotary_half_kv_write);
+  m.def("parallel_add_norm_f32", &parallel_add_norm_f32);
   m.def("latent_norm_write", &latent_norm_write);
   m.def("hyper_connect", &hyper_connect);
   m.def("head_linear", &head_linear);

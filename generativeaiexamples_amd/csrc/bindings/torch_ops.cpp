@@ -379,15 +379,20 @@ void sim_topk(const Tensor& Q, const Tensor& X, const Tensor& bias, int64_t n_ro
 
 void moe_route(const Tensor& logits, int64_t k, bool renorm, Tensor& ids, Tensor& w, bool sigmoid,
                const optional<Tensor>& bias, double eps) {
-  check_f32(logits, "router logits");
+  check_dev(logits, "router logits");  // rows may be a column slice of a wider projection
+  TORCH_CHECK(logits.scalar_type() == at::kFloat && logits.dim() == 2 && (logits.stride(1) == 1 || logits.size(1) == 1),
+              "moe_route: fp32 logits [T, E] with contiguous rows");
   check_i32(ids, "topk ids");
   check_f32(w, "topk weights");
+  TORCH_CHECK(ids.is_contiguous() && w.is_contiguous() && ids.numel() == logits.size(0) * k && w.numel() == ids.numel(),
+              "moe_route: ids / w [T, k]");
   if (bias) {
     check_f32(*bias, "choice bias");
     TORCH_CHECK(bias->is_contiguous() && bias->numel() == logits.size(1) && !sigmoid, "moe_route: bias [E], softmax scoring");
   }
   gai_moe_route(logits.data_ptr<float>(), logits.size(0), logits.size(1), k, renorm ? 1 : 0, ids.data_ptr<int>(),
-                w.data_ptr<float>(), cur_stream(), sigmoid ? 1 : 0, bias ? bias->data_ptr<float>() : nullptr, (float)eps);
+                w.data_ptr<float>(), cur_stream(), sigmoid ? 1 : 0, bias ? bias->data_ptr<float>() : nullptr, (float)eps,
+                (int)logits.stride(0));
 }
 
 void moe_scale_rows(const Tensor& h, const Tensor& pos, const Tensor& w, Tensor& out) {

@@ -142,7 +142,7 @@ int gai_moe_gemm_dec2(const void* A, const int* a_rows, const void* W, void* C, 
                       int rows_total, int N, int K, int act, hipStream_t st, float actp = 0.f);
 // sigmoid: scores sigmoid(logit) per expert instead of a softmax over the experts (weights = the chosen scores)
 void gai_moe_route(const float* logits, int T, int E, int k, int renorm, int* ids, float* w, hipStream_t st,
-                   int sigmoid = 0, const float* bias = nullptr, float eps = 0.f);
+                   int sigmoid = 0, const float* bias = nullptr, float eps = 0.f, int ld = 0);  // ld: row stride (0: E)
 // dt: 0 bf16 (MFMA tiles when K % 64 == 0), 1 fp32 (generic grouped kernel, true fp32)
 void gai_moe_gemm(const void* A, const int* a_rows, const void* W, void* C, const int* offs, int E, int rows_total,
                   int N, int K, int act, hipStream_t st, int dt = 0, float actp = 0.f);
@@ -249,17 +249,18 @@ void gai_window_attention(const void* q, const void* k_cache, const void* v_cach
                           float scale, float softcap, int window, const float* r1, const float* r2, const void* gate,
                           int ldg, const float* sig_bias, int sig, float out_scale, int dt, hipStream_t st,
                           float* part = nullptr, int chunk = 0, const float* hscale = nullptr, int has_sink = 0,
-                          float sink = 0.f, const float* hsink = nullptr);
+                          float sink = 0.f, const float* hsink = nullptr, int ghead = 0);  // ghead: one gate per head
 // q_out = rmsnorm(dq) * wq; K page row and V^T page (one kv head, key and value size R) = rmsnorm(dkv) * wkv
 void gai_latent_norm_write(const void* dq, int ldq, const float* wq, const void* dkv, int ldk, const float* wkv,
                            const int* slots, void* q_out, void* k_cache, void* v_cache, int T, int RQ, int R, float eps,
                            int dt, hipStream_t st);
-// attention_mqa.hip: bf16 softmax attention with one kv head shared by all heads, optional window and sinks per head
-int gai_mqa_attention_ok(int DK, int DV);
-size_t gai_mqa_attention_ws_floats(int T, int S, int H, int DV);
-void gai_mqa_attention(const void* q, const void* k_cache, const void* v_cache, const int* block_tables, int maxb,
-                       const int* cu_q, const int* ctx, int S, void* out, int ldo, int T, int H, int DK, int DV, float scale,
-                       int window, const float* sink, float* ws, hipStream_t st);
+// attention_gqa.hip: bf16 softmax attention with kv heads shared by groups of heads, optional window, sinks and output
+// gates (one per head)
+int gai_gqa_attention_ok(int DK, int DV);
+size_t gai_gqa_attention_ws_floats(int T, int S, int H, int G, int DV);
+void gai_gqa_attention(const void* q, const void* k_cache, const void* v_cache, const int* block_tables, int maxb,
+                       const int* cu_q, const int* ctx, int S, void* out, int ldo, int T, int H, int G, int DK, int DV,
+                       float scale, int window, const float* sink, const void* gate, int ldg, float* ws, hipStream_t st);
 // hyper.hip: close one sublayer of a hyper-connected decoder (streams X, output y) and open the next (layer norm)
 void gai_hyper_connect(float* X, const float* x0, const void* y, int ldy, const float* mix, const float* out_w,
                        const float* in_w, const float* norm_w, void* out, int T, int ns, int D, float eps, int dt_y,
@@ -277,6 +278,14 @@ void gai_mlstm(const void* q, int ldq, const void* k, int ldk, const void* v, in
 void gai_rotary_kv_write(const void* q, int ldq, const void* k, int ldk, const void* v, int ldv, const int* positions,
                          const int* slots, void* q_out, void* k_cache, void* v_cache, int T, int H, int G, int DK, int DV,
                          int ROT, float base, int dt_in, int dt, hipStream_t st);
+// rotate-half positions (inv_freq: fp64 [half]), unit RMS norm per head (unit_eps >= 0), cache write
+void gai_rotary_half_kv_write(const void* q, int ldq, const void* k, int ldk, const void* v, int ldv, const int* positions,
+                              const int* slots, void* q_out, void* k_cache, void* v_cache, int T, int H, int G, int DK,
+                              int DV, const double* inv_freq, int half, float unit_eps, int dt, hipStream_t st);
+// norm_f32.hip: res += sa * a + sb * b; h1 / h2 = rmsnorm(res) * w1 / w2 (every pointer but res optional)
+void gai_parallel_add_norm_f32(float* res, const void* a, int lda, const float* sa, const void* b, int ldb, const float* sb,
+                               const float* w1, void* h1, const float* w2, void* h2, int T, int D, float eps, int dt,
+                               hipStream_t st);
 // sigmoid-mode decode steps: number of key splits (1: none); part must hold splits * T * H * DV floats
 int gai_sigmoid_attention_splits(int T, int S, int H);
 // recurrent.hip

@@ -1,21 +1,21 @@
-// Paged softmax attention with ONE kv head shared by all query heads (latent attention over the cached latent, multi-query
-// attention), bf16 pages, fp32 scores, weights and sums:
+// Paged softmax attention whose query heads share kv heads (grouped-query, multi-query, latent attention over the cached
+// latent), bf16 pages, fp32 scores, weights and sums:
 //
 //   s_ij = scale * (q_i . k_j),  j <= i (and i - j < window when window > 0)
-//   o_i  = sum_j e^(s_ij) v_j / (sum_j e^(s_ij) + e^(sink_h))
+//   o_i  = sigmoid(gate_ih) sum_j e^(s_ij) v_j / (sum_j e^(s_ij) + e^(sink_h))      (gate, sink: optional, one per head)
 //
-// All heads of a token see the same keys, so a "row" here is a (token, head) pair of q viewed as [T * H, DK] and the matrix-core
-// tile is 32 such rows (two tokens of 16 heads, say) against 32 keys. S^T = K.Q^T on v_mfma_f32_32x32x16_bf16 leaves one row per
+// The R = H / G query heads of one kv head see the same keys, so a "row" here is a (token, head of the group) pair and the
+// matrix-core tile is 32 such rows (eight tokens of four heads, say) against 32 keys of that kv head (blockIdx.z). S^T = K.Q^T on v_mfma_f32_32x32x16_bf16 leaves one row per
 // lane; the softmax is in-register fp32; P.V runs on the same MFMA with the fp32 weights split into two bf16 terms. K row
 // pi(i) feeds accumulator row i with pi = swap of bits 2 and 3, so that the eight weights a lane holds for a 16-key step are
 // eight consecutive keys: the V^T fragment is one 16-byte load. The running maximum is allowed to lag by 2^8 before the
 // accumulators are rescaled (the weights stay within fp32 and the final division cancels the factor), so rescaling is rare.
 //
-// mqa_prefill_kernel: NW waves of a workgroup (32 NW consecutive rows of a sequence) share 32-key blocks staged in LDS by
+// gqa_prefill_kernel: NW waves of a workgroup (32 NW consecutive rows of a sequence) share 32-key blocks staged in LDS by
 // direct global -> LDS loads, double buffered; both images are XOR-swizzled through the per-lane source address so that
 // fragment reads are conflict-free. Long tiles are launched first (causal rows differ in length).
-// mqa_split_kernel: sequences with few rows (decoded tokens, short portions): one wave per (32 rows, share of the key blocks),
-// fragments straight from memory; partial sums, maxima and denominators are merged by mqa_merge_kernel.
+// gqa_split_kernel: sequences with few rows (decoded tokens, short portions): one wave per (32 rows, share of the key blocks),
+// fragments straight from memory; partial sums, maxima and denominators are merged by gqa_merge_kernel.
 #include "gai_common.h"
 #include "gai_kernels.h"
 
@@ -29,18 +29,21 @@ constexpr float kLag = 8.f;        // how far (powers of two) the running maximu
 constexpr int kShortRows = 128;    // sequences of fewer rows go to the key-split kernel
 constexpr int kMaxSplit = 32;
 
-struct MqaArgs {
+struct GqaArgs {
   const bf16 *q, *kc, *vc;
   const int *bt, *cu, *ctx;
-  int maxb, S, T, H;
+  int maxb, S, T, H, G, R;         // R = H / G query heads per kv head
   float scale2;                    // scale * log2(e)
   int window;
   const float* sink;               // [H] or null
+  const bf16* gate;                // [T, >= H] or null
+  int ldg;
   bf16* out;
   int ldo;
-  float* part;                     // [nsplit][T * H][DV + 4]: sums, maximum (log2 units), denominator
+  float* part;                     // [nsplit][S * G * prow][DV + 4]: sums, maximum (log2 units), denominator
   int nsplit;
   int tps;                         // tiles of 32 rows per sequence in the key-split launch
+  int prow;                        // rows per (sequence, kv head) in part
 };
 
 __device__ __forceinline__ int key_perm(int i) { return (i & 0x13) | ((i & 4) << 1) | ((i & 8) >> 1); }
@@ -98,6 +101,10 @@ __device__ __forceinline__ void soft_block(f32x16& sc, float scale2, bool masked
   l += rs;
 }
 
+__device__ __forceinline__ float head_gate(const GqaArgs& a, int t, int head) {
+  return 1.0f / (1.0f + __expf(-(float)a.gate[(size_t)t * a.ldg + head]));
+}
+
 __device__ __forceinline__ void split_weights(const f32x16& sc, int ks, bf16x8& hi, bf16x8& lo) {
 #pragma unroll
   for (int e = 0; e < 8; ++e) {
@@ -108,35 +115,36 @@ __device__ __forceinline__ void split_weights(const f32x16& sc, int ks, bf16x8& 
 }
 
 template <int DK, int DV, int NW>
-__global__ __launch_bounds__(64 * NW) void mqa_prefill_kernel(MqaArgs a) {
+__global__ __launch_bounds__(64 * NW) void gqa_prefill_kernel(GqaArgs a) {
   constexpr int KB = 32 * DK * 2, VB = 32 * DV * 2, KI = KB / 1024, VI = VB / 1024;  // staged bytes / 1-KiB loads per block
   extern __shared__ __attribute__((aligned(16))) char smem[];                          // [2][K | V]
   const int tid = threadIdx.x, wv = tid >> 6, lane = tid & 63, qi = lane & 31, hb = lane >> 5;
   // ---- tile -> (sequence, first row); the last tiles of the launch first
   int total = 0;
   for (int s = 0; s < a.S; ++s) {
-    const int rows = (a.cu[s + 1] - a.cu[s]) * a.H;
+    const int rows = (a.cu[s + 1] - a.cu[s]) * a.R;
     total += rows >= kShortRows ? (rows + 32 * NW - 1) / (32 * NW) : 0;
   }
   if ((int)blockIdx.x >= total) return;
   int tile = total - 1 - (int)blockIdx.x, s = 0, rows = 0;
   for (; s < a.S; ++s) {
-    rows = (a.cu[s + 1] - a.cu[s]) * a.H;
+    rows = (a.cu[s + 1] - a.cu[s]) * a.R;
     const int n = rows >= kShortRows ? (rows + 32 * NW - 1) / (32 * NW) : 0;
     if (tile < n) break;
     tile -= n;
   }
   const int len = a.cu[s + 1] - a.cu[s], c0 = a.ctx[s] - len;   // position of the portion's first token
   const int r_wg = tile * 32 * NW, r_wv = r_wg + 32 * wv, row = min(r_wv + qi, rows - 1);
-  const int pos = c0 + row / a.H;
-  const int p_first = c0 + min(r_wv, rows - 1) / a.H, p_last = c0 + min(r_wv + 31, rows - 1) / a.H;  // of this wave
-  const int wg_first = c0 + r_wg / a.H, wg_last = c0 + min(r_wg + 32 * NW - 1, rows - 1) / a.H;
+  const int pos = c0 + row / a.R;
+  const int p_first = c0 + min(r_wv, rows - 1) / a.R, p_last = c0 + min(r_wv + 31, rows - 1) / a.R;  // of this wave
+  const int wg_first = c0 + r_wg / a.R, wg_last = c0 + min(r_wg + 32 * NW - 1, rows - 1) / a.R;
   const int kb0 = (a.window > 0 ? max(0, wg_first - a.window + 1) : 0) & ~31;
   const int lo = a.window > 0 ? pos - a.window + 1 : 0;
   const int lo_first = a.window > 0 ? p_first - a.window + 1 : 0, lo_last = a.window > 0 ? p_last - a.window + 1 : 0;
   const bool live = r_wv < rows;
   const int* bt = a.bt + (size_t)s * a.maxb;
-  const bf16* qr = a.q + ((size_t)a.cu[s] * a.H + row) * DK + 8 * hb;
+  const int g = blockIdx.z, t = a.cu[s] + row / a.R, head = g * a.R + row % a.R;
+  const bf16* qr = a.q + ((size_t)t * a.H + head) * DK + 8 * hb;
   bf16x8 qf[DK / 16];
 #pragma unroll
   for (int i = 0; i < DK / 16; ++i) qf[i] = load8(qr + 16 * i);
@@ -148,13 +156,13 @@ __global__ __launch_bounds__(64 * NW) void mqa_prefill_kernel(MqaArgs a) {
 #pragma unroll
     for (int i = wv; i < KI; i += NW) {
       const int slot = 64 * i + lane, r = slot / (DK / 8), ch = (slot % (DK / 8)) ^ k_swz<DK>(r);
-      const bf16* src = a.kc + ((size_t)(r < 16 ? pg0 : pg1) * 16 + (r & 15)) * DK + 8 * ch;
+      const bf16* src = a.kc + (((size_t)(r < 16 ? pg0 : pg1) * a.G + g) * 16 + (r & 15)) * DK + 8 * ch;
       __builtin_amdgcn_global_load_lds(src, GAI_LDS(kd + i * 1024), 16, 0, 0);
     }
 #pragma unroll
     for (int i = wv; i < VI; i += NW) {
       const int slot = 64 * i + lane, pg = slot / (2 * DV), c = (slot % (2 * DV)) >> 1, hf = (slot & 1) ^ ((c >> 3) & 1);
-      const bf16* src = a.vc + ((size_t)(pg ? pg1 : pg0) * DV + c) * 16 + 8 * hf;
+      const bf16* src = a.vc + (((size_t)(pg ? pg1 : pg0) * a.G + g) * DV + c) * 16 + 8 * hf;
       __builtin_amdgcn_global_load_lds(src, GAI_LDS(vd + i * 1024), 16, 0, 0);
     }
   };
@@ -198,13 +206,13 @@ __global__ __launch_bounds__(64 * NW) void mqa_prefill_kernel(MqaArgs a) {
   if (r_wv + qi >= rows) return;
   float f = 1.0f;
   if (a.sink) {
-    const float sk = a.sink[row % a.H] * kL2e, mf = fmaxf(m, sk);
+    const float sk = a.sink[head] * kL2e, mf = fmaxf(m, sk);
     f = __builtin_amdgcn_exp2f(m - mf);
     l = l * f + __builtin_amdgcn_exp2f(sk - mf);
   }
   f /= l;
-  const int t = a.cu[s] + row / a.H;
-  bf16* o = a.out + (size_t)t * a.ldo + (size_t)(row % a.H) * DV;
+  if (a.gate) f *= head_gate(a, t, head);
+  bf16* o = a.out + (size_t)t * a.ldo + (size_t)head * DV;
 #pragma unroll
   for (int i = 0; i < DV / 32; ++i)
 #pragma unroll
@@ -216,27 +224,27 @@ __global__ __launch_bounds__(64 * NW) void mqa_prefill_kernel(MqaArgs a) {
     }
 }
 
-// blockIdx.x = sequence * tps + tile of 32 rows, blockIdx.y = share of the key blocks
+// blockIdx.z = kv head, blockIdx.x = sequence * tps + tile of 32 rows, blockIdx.y = share of the key blocks
 template <int DK, int DV>
-__global__ __launch_bounds__(64) void mqa_split_kernel(MqaArgs a) {
+__global__ __launch_bounds__(64) void gqa_split_kernel(GqaArgs a) {
   const int lane = threadIdx.x, qi = lane & 31, hb = lane >> 5;
   const int s = blockIdx.x / a.tps, r0 = (blockIdx.x % a.tps) * 32;
-  const int len = a.cu[s + 1] - a.cu[s], rows = len * a.H;
-  if (rows >= kShortRows || r0 >= rows) return;
+  const int len = a.cu[s + 1] - a.cu[s], rows = len * a.R;
+  if (rows >= kShortRows || rows > a.prow || r0 >= rows) return;
   const int c0 = a.ctx[s] - len, row = min(r0 + qi, rows - 1);
-  const int pos = c0 + row / a.H, p_first = c0 + r0 / a.H, p_last = c0 + min(r0 + 31, rows - 1) / a.H;
+  const int pos = c0 + row / a.R, p_first = c0 + r0 / a.R, p_last = c0 + min(r0 + 31, rows - 1) / a.R;
   const int lo = a.window > 0 ? pos - a.window + 1 : 0, lo_last = a.window > 0 ? p_last - a.window + 1 : 0;
   int kb0 = (a.window > 0 ? max(0, p_first - a.window + 1) : 0) & ~31;
   const int nblk = (p_last - kb0) / 32 + 1, per = (nblk + a.nsplit - 1) / a.nsplit;
   kb0 += (int)blockIdx.y * per * 32;
   const int kb1 = min(p_last, kb0 + per * 32 - 1);
   const int* bt = a.bt + (size_t)s * a.maxb;
-  const size_t g_row = (size_t)a.cu[s] * a.H + row;
-  float* po = a.part + ((size_t)blockIdx.y * a.T * a.H + g_row) * (DV + 4);
+  const int g = blockIdx.z;
+  float* po = a.part + (((size_t)blockIdx.y * a.S + s) * a.G + g) * a.prow * (DV + 4) + (size_t)row * (DV + 4);
   const bool mine = r0 + qi < rows;
   float m = kOut, l = 0.f;
   if (kb0 > kb1) return;  // no key block left for this share: the merge does not read it
-  const bf16* qr = a.q + g_row * DK + 8 * hb;
+  const bf16* qr = a.q + ((size_t)(a.cu[s] + row / a.R) * a.H + g * a.R + row % a.R) * DK + 8 * hb;
   bf16x8 qf[DK / 16];
 #pragma unroll
   for (int i = 0; i < DK / 16; ++i) qf[i] = load8(qr + 16 * i);
@@ -246,14 +254,14 @@ __global__ __launch_bounds__(64) void mqa_split_kernel(MqaArgs a) {
   const int kr = key_perm(qi), lp = p_last >> 4;
   for (int kb = kb0; kb <= kb1; kb += 32) {
     const int pg[2] = {bt[kb >> 4], bt[min((kb >> 4) + 1, lp)]};
-    const bf16* kp = a.kc + ((size_t)(kr < 16 ? pg[0] : pg[1]) * 16 + (kr & 15)) * DK + 8 * hb;
+    const bf16* kp = a.kc + (((size_t)(kr < 16 ? pg[0] : pg[1]) * a.G + g) * 16 + (kr & 15)) * DK + 8 * hb;
     bf16x8 kf[DK / 16], vf[2][DV / 32];  // the values of the block are on their way while it is scored
 #pragma unroll
     for (int i = 0; i < DK / 16; ++i) kf[i] = load8(kp + 16 * i);
 #pragma unroll
     for (int k2 = 0; k2 < 2; ++k2)
 #pragma unroll
-      for (int i = 0; i < DV / 32; ++i) vf[k2][i] = load8(a.vc + ((size_t)pg[k2] * DV + qi) * 16 + 8 * hb + 32 * i * 16);
+      for (int i = 0; i < DV / 32; ++i) vf[k2][i] = load8(a.vc + (((size_t)pg[k2] * a.G + g) * DV + qi) * 16 + 8 * hb + 32 * i * 16);
     f32x16 sc = f32x16{};
 #pragma unroll
     for (int i = 0; i < DK / 16; ++i) sc = __builtin_amdgcn_mfma_f32_32x32x16_bf16(kf[i], qf[i], sc, 0, 0, 0);
@@ -283,34 +291,33 @@ __global__ __launch_bounds__(64) void mqa_split_kernel(MqaArgs a) {
   }
 }
 
-// one wave per row (blockIdx.x) of every short sequence (blockIdx.y)
+// one wave per row (blockIdx.x) of every short sequence (blockIdx.y), blockIdx.z = kv head
 template <int DV>
-__global__ __launch_bounds__(64) void mqa_merge_kernel(MqaArgs a) {
+__global__ __launch_bounds__(64) void gqa_merge_kernel(GqaArgs a) {
   __shared__ float wgt[kMaxSplit];
   const int s = blockIdx.y, row = blockIdx.x, lane = threadIdx.x;
-  const int rows = (a.cu[s + 1] - a.cu[s]) * a.H;
-  if (rows >= kShortRows || row >= rows) return;
-  const size_t g_row = (size_t)a.cu[s] * a.H + row, TH = (size_t)a.T * a.H;
-  const float* p0 = a.part + g_row * (DV + 4);
-  const size_t step = TH * (DV + 4);
+  const int rows = (a.cu[s + 1] - a.cu[s]) * a.R;
+  if (rows >= kShortRows || rows > a.prow || row >= rows) return;
+  const int g = blockIdx.z, t = a.cu[s] + row / a.R, head = g * a.R + row % a.R;
+  const float* p0 = a.part + (((size_t)s * a.G + g) * a.prow + row) * (DV + 4);
+  const size_t step = (size_t)a.S * a.G * a.prow * (DV + 4);
   // the shares that held key blocks of this row's tile, as the key-split kernel dealt them out
   const int len = a.cu[s + 1] - a.cu[s], c0 = a.ctx[s] - len, r0 = row & ~31;
-  const int k_lo = (a.window > 0 ? max(0, c0 + r0 / a.H - a.window + 1) : 0) & ~31;
-  const int nblk = (c0 + min(r0 + 31, rows - 1) / a.H - k_lo) / 32 + 1, per = (nblk + a.nsplit - 1) / a.nsplit;
+  const int k_lo = (a.window > 0 ? max(0, c0 + r0 / a.R - a.window + 1) : 0) & ~31;
+  const int nblk = (c0 + min(r0 + 31, rows - 1) / a.R - k_lo) / 32 + 1, per = (nblk + a.nsplit - 1) / a.nsplit;
   const int used = (nblk + per - 1) / per;
   float m = kOut, l = 0.f;
   if (lane < used) {
     m = p0[lane * step + DV];
     l = p0[lane * step + DV + 1];
   }
-  const float sk = a.sink ? a.sink[row % a.H] * kL2e : kOut;
+  const float sk = a.sink ? a.sink[head] * kL2e : kOut;
   const float M = fmaxf(wave_max(m), sk);
   const float w = l > 0.f ? __builtin_amdgcn_exp2f(m - M) : 0.f;
   const float den = wave_sum(l * w) + (a.sink ? __builtin_amdgcn_exp2f(sk - M) : 0.f);
-  if (lane < used) wgt[lane] = w / den;
+  if (lane < used) wgt[lane] = w / den * (a.gate ? head_gate(a, t, head) : 1.0f);
   __syncthreads();
-  const int t = a.cu[s] + row / a.H;
-  bf16* o = a.out + (size_t)t * a.ldo + (size_t)(row % a.H) * DV;
+  bf16* o = a.out + (size_t)t * a.ldo + (size_t)head * DV;
   for (int c = 4 * lane; c < DV; c += 256) {
     f32x4 y = f32x4{0.f, 0.f, 0.f, 0.f};
 #pragma unroll 8
@@ -319,61 +326,66 @@ __global__ __launch_bounds__(64) void mqa_merge_kernel(MqaArgs a) {
   }
 }
 
-int tiles_per_seq(int T, int S, int H) { return T == S ? (H + 31) / 32 : kShortRows / 32; }
+int tiles_per_seq(int T, int S, int R) { return T == S ? (R + 31) / 32 : kShortRows / 32; }
 
-int split_count(int T, int S, int H) {
-  const int tiles = S * (T == S ? (H + 31) / 32 : (T / S < 4 ? T / S * H + 31 : kShortRows) / 32);
-  int n = 1024 / (tiles < 1 ? 1 : tiles);
-  return n < 4 ? 4 : (n > kMaxSplit ? kMaxSplit : n);
+int split_count(int T, int S, int R, int G) {
+  const long tiles = (long)S * G * ((T == S ? R + 31 : (T / S < 4 ? T / S * R + 31 : kShortRows)) / 32);
+  const long n = 1024 / (tiles < 1 ? 1 : tiles);
+  return n < 4 ? 4 : (n > kMaxSplit ? kMaxSplit : (int)n);
 }
 
+int part_rows(int T, int S, int R) { return T == S ? R : kShortRows; }
+
 template <int DK, int DV>
-void launch(const MqaArgs& a, hipStream_t st) {
-  const long TH = (long)a.T * a.H;
-  if (a.T > a.S || a.H >= kShortRows) {
+void launch(const GqaArgs& a, hipStream_t st) {
+  const long rows = (long)a.T * a.R;   // of one kv head
+  if (a.T > a.S || a.R >= kShortRows) {
     constexpr size_t lds = 2 * 32 * (DK + DV) * 2;
-    const int g8 = (int)(TH / 256) + a.S;
-    if (TH >= 256 * 256) {
+    if (rows * a.G >= 256 * 256) {
       if (lds > 64 * 1024)
-        (void)hipFuncSetAttribute(reinterpret_cast<const void*>(mqa_prefill_kernel<DK, DV, 8>),
+        (void)hipFuncSetAttribute(reinterpret_cast<const void*>(gqa_prefill_kernel<DK, DV, 8>),
                                   hipFuncAttributeMaxDynamicSharedMemorySize, 160 * 1024);
-      mqa_prefill_kernel<DK, DV, 8><<<g8, 512, lds, st>>>(a);
+      gqa_prefill_kernel<DK, DV, 8><<<dim3((int)(rows / 256) + a.S, 1, a.G), 512, lds, st>>>(a);
     } else {
       if (lds > 64 * 1024)
-        (void)hipFuncSetAttribute(reinterpret_cast<const void*>(mqa_prefill_kernel<DK, DV, 4>),
+        (void)hipFuncSetAttribute(reinterpret_cast<const void*>(gqa_prefill_kernel<DK, DV, 4>),
                                   hipFuncAttributeMaxDynamicSharedMemorySize, 160 * 1024);
-      mqa_prefill_kernel<DK, DV, 4><<<(int)(TH / 128) + a.S, 256, lds, st>>>(a);
+      gqa_prefill_kernel<DK, DV, 4><<<dim3((int)(rows / 128) + a.S, 1, a.G), 256, lds, st>>>(a);
     }
   }
-  if (a.H < kShortRows) {
-    mqa_split_kernel<DK, DV><<<dim3(a.tps * a.S, a.nsplit), 64, 0, st>>>(a);
-    mqa_merge_kernel<DV><<<dim3(32 * a.tps, a.S), 64, 0, st>>>(a);
+  if (a.R < kShortRows) {
+    gqa_split_kernel<DK, DV><<<dim3(a.tps * a.S, a.nsplit, a.G), 64, 0, st>>>(a);
+    gqa_merge_kernel<DV><<<dim3(a.prow, a.S, a.G), 64, 0, st>>>(a);
   }
 }
 
 }  // namespace
 
 // 1: the key / value sizes have matrix-core kernels here
-int gai_mqa_attention_ok(int DK, int DV) {
+int gai_gqa_attention_ok(int DK, int DV) {
   return (DK == DV && (DK == 32 || DK == 64 || DK == 96 || DK == 128 || DK == 160 || DK == 192 || DK == 256)) ||
-         (DK == 96 && DV == 64) || (DK == 192 && DV == 128);
+         (DK == 96 && DV == 64) || (DK == 192 && DV == 128) || (DK == 64 && DV == 128) || (DK == 128 && DV == 64);
 }
 
-size_t gai_mqa_attention_ws_floats(int T, int S, int H, int DV) {
-  return H < kShortRows && T > 0 && S > 0 ? (size_t)split_count(T, S, H) * T * H * (DV + 4) : 0;
+size_t gai_gqa_attention_ws_floats(int T, int S, int H, int G, int DV) {
+  const int R = H / G;
+  return R < kShortRows && T > 0 && S > 0 ? (size_t)split_count(T, S, R, G) * S * G * part_rows(T, S, R) * (DV + 4) : 0;
 }
 
-void gai_mqa_attention(const void* q, const void* k_cache, const void* v_cache, const int* block_tables, int maxb,
-                       const int* cu_q, const int* ctx, int S, void* out, int ldo, int T, int H, int DK, int DV, float scale,
-                       int window, const float* sink, float* ws, hipStream_t st) {
+void gai_gqa_attention(const void* q, const void* k_cache, const void* v_cache, const int* block_tables, int maxb,
+                       const int* cu_q, const int* ctx, int S, void* out, int ldo, int T, int H, int G, int DK, int DV,
+                       float scale, int window, const float* sink, const void* gate, int ldg, float* ws, hipStream_t st) {
   if (T == 0 || S == 0) return;
-  if (ldo % 4) gai_launch_error(__FILE__, __LINE__, "mqa_attention: output rows on a grid of four elements");
-  const MqaArgs a{(const bf16*)q, (const bf16*)k_cache, (const bf16*)v_cache, block_tables, cu_q, ctx, maxb, S, T, H,
-                  scale * kL2e, window, sink, (bf16*)out, ldo, ws, split_count(T, S, H), tiles_per_seq(T, S, H)};
-  if (H < kShortRows && !ws) gai_launch_error(__FILE__, __LINE__, "mqa_attention: scratch missing");
-#define GAI_MQA(K_, V_) if (DK == K_ && DV == V_) { launch<K_, V_>(a, st); GAI_LAUNCH_CHECK(); return; }
-  GAI_MQA(32, 32) GAI_MQA(64, 64) GAI_MQA(96, 96) GAI_MQA(128, 128) GAI_MQA(160, 160) GAI_MQA(192, 192) GAI_MQA(256, 256)
-  GAI_MQA(96, 64) GAI_MQA(192, 128)
-#undef GAI_MQA
-  gai_launch_error(__FILE__, __LINE__, "mqa_attention: no kernel for these key / value sizes");
+  if (G < 1 || H % G) gai_launch_error(__FILE__, __LINE__, "gqa_attention: heads must be a multiple of kv heads");
+  if (ldo % 4) gai_launch_error(__FILE__, __LINE__, "gqa_attention: output rows on a grid of four elements");
+  const int R = H / G;
+  const GqaArgs a{(const bf16*)q, (const bf16*)k_cache, (const bf16*)v_cache, block_tables, cu_q, ctx, maxb, S, T, H, G, R,
+                  scale * kL2e, window, sink, (const bf16*)gate, ldg, (bf16*)out, ldo, ws, split_count(T, S, R, G),
+                  tiles_per_seq(T, S, R), part_rows(T, S, R)};
+  if (R < kShortRows && !ws) gai_launch_error(__FILE__, __LINE__, "gqa_attention: scratch missing");
+#define GAI_GQA(K_, V_) if (DK == K_ && DV == V_) { launch<K_, V_>(a, st); GAI_LAUNCH_CHECK(); return; }
+  GAI_GQA(32, 32) GAI_GQA(64, 64) GAI_GQA(96, 96) GAI_GQA(128, 128) GAI_GQA(160, 160) GAI_GQA(192, 192) GAI_GQA(256, 256)
+  GAI_GQA(96, 64) GAI_GQA(192, 128) GAI_GQA(64, 128) GAI_GQA(128, 64)
+#undef GAI_GQA
+  gai_launch_error(__FILE__, __LINE__, "gqa_attention: no kernel for these key / value sizes");
 }

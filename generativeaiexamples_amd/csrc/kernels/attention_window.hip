@@ -3,7 +3,8 @@
 //   s_ij = cap * tanh(scale * (q_i . k_j) / cap) - r1_h * ln(1 + r2_h * (i - j)),   0 <= i - j < window
 //   o_i  = softmax_j(s_ij) V
 //
-// optionally times sigmoid(gate_i) element by element (an output gate read from the same projection as q, k, v).
+// optionally times sigmoid(gate_i), an element or (ghead) a head at a time (an output gate read from the same projection
+// as q, k, v).
 // (cap <= 0: no cap; r1 = nullptr: no distance term; window <= 0: plain causal.) Positions enter only through the
 // distance term and the window: there is no rotation. K / V live in the engine's paged cache (16-token pages,
 // K [page, G, 16, DK], V^T [page, G, DV, 16]) in bf16 or fp32; scores, softmax weights and the P.V sums are fp32.
@@ -21,6 +22,10 @@
 // rotary_kv_write: rotation of the channel pairs (2i, 2i + 1), i < ROT / 2, of every q and k head by position *
 // base^(-2i / ROT) (the rest of a head passes unchanged), then q -> q_out and k, v -> their cache slots. The angle is
 // formed and reduced to (-pi, pi] in fp64, sine and cosine are libm sincosf of the reduced angle.
+//
+// rotary_half_kv_write: rotation of the channel pairs (i, i + half), i < half, of every q and k head by position *
+// inv_freq[i] (fp64 table; the angle is formed and reduced in fp64), then (unit_eps >= 0) every q and k head divided by its
+// root mean square, then q -> q_out and k, v -> their cache slots; one wave64 per head.
 //
 // headnorm_kv_write: RMS norm of every q head and every k head over its own DK channels (one weight vector of size DK
 // shared by the heads), optionally times a query temperature 1 + coef * ln(floor((p + 1) / every) + 1) of the token's
@@ -345,6 +350,99 @@ __global__ __launch_bounds__(256) void rotary_kv_write_kernel(const TI* __restri
   }
 }
 
+// Workgroups of the first nqk: q and k heads of one token, a wave per head (up to 64 NJ groups of VEC channels in
+// registers); the others: v of VT tokens, a thread per channel, so that tokens filling a whole page store its V^T row at once.
+constexpr int kHalfRegs = 8;
+
+template <typename TA, int VEC, int VT>
+__global__ __launch_bounds__(256) void rotary_half_kv_write_kernel(
+    const TA* __restrict__ q, int ldq, const TA* __restrict__ k, int ldk, const TA* __restrict__ v, int ldv,
+    const int* __restrict__ positions, const int* __restrict__ slots, TA* __restrict__ q_out, TA* __restrict__ k_cache,
+    TA* __restrict__ v_cache, int T, int H, int G, int DK, int DV, const double* __restrict__ inv_freq, int half,
+    float unit_eps) {
+  const int tid = threadIdx.x;
+  if ((int)blockIdx.x >= T) {
+    const int t0 = ((int)blockIdx.x - T) * VT, n = min(VT, T - t0), NV = G * DV, s0 = slots[t0];
+    const bool page = VT == 16 && n == 16 && (s0 & 15) == 0 && __all(slots[t0 + (tid & 15)] == s0 + (tid & 15));
+    for (int i = tid; i < NV; i += 256) {
+      const int g = i / DV, c = i - g * DV;
+      const TA* src = v + (size_t)t0 * ldv + i;
+      if (page) {
+        TA* dst = v_cache + (((size_t)(s0 >> 4) * G + g) * DV + c) * 16;
+        __attribute__((aligned(16))) TA x[16];
+#pragma unroll
+        for (int j = 0; j < 16; ++j) x[j] = src[(size_t)j * ldv];
+#pragma unroll
+        for (int j = 0; j < (int)sizeof(TA); ++j)
+          reinterpret_cast<uint4*>(dst)[j] = reinterpret_cast<const uint4*>(x)[j];
+      } else {
+        for (int j = 0; j < n; ++j) {
+          const int s = slots[t0 + j];
+          v_cache[(((size_t)(s >> 4) * G + g) * DV + c) * 16 + (s & 15)] = src[(size_t)j * ldv];
+        }
+      }
+    }
+    return;
+  }
+  extern __shared__ float cs[];  // cos[half] | sin[half]
+  const int t = blockIdx.x, wid = tid >> 6, lane = tid & 63;
+  const double pos = (double)positions[t];
+  for (int i = tid; i < half; i += 256) {
+    const double a = pos * inv_freq[i];
+    const double r = a - 6.283185307179586476925 * rint(a * 0.15915494309189533577);
+    float sn, c;
+    sincosf((float)r, &sn, &c);
+    cs[i] = c;
+    cs[half + i] = sn;
+  }
+  __syncthreads();
+  const int slot = slots[t], off = slot & 15;
+  const size_t page = slot >> 4;
+  typedef TA vec __attribute__((ext_vector_type(VEC)));
+  for (int hh = wid; hh < H + G; hh += 4) {  // q heads, then k heads: wave-uniform
+    const bool isq = hh < H;
+    const int g = isq ? hh : hh - H;
+    const TA* src = isq ? q + (size_t)t * ldq + (size_t)g * DK : k + (size_t)t * ldk + (size_t)g * DK;
+    TA* dst = isq ? q_out + ((size_t)t * H + g) * DK : k_cache + ((page * G + g) * 16 + off) * DK;
+    float y[kHalfRegs][VEC];
+    float ss = 0.f;
+#pragma unroll
+    for (int r = 0; r < kHalfRegs; ++r) {
+      const int i = (lane + 64 * r) * VEC;
+      if (i < DK) {
+        const vec x = *reinterpret_cast<const vec*>(src + i);
+        if (i < 2 * half) {   // VEC divides half: the group has one partner group
+          const bool up = i >= half;
+          const vec p = *reinterpret_cast<const vec*>(src + (up ? i - half : i + half));
+          const int f = up ? i - half : i;
+#pragma unroll
+          for (int e = 0; e < VEC; ++e) {
+            const float c = cs[f + e], sn = cs[half + f + e];
+            y[r][e] = up ? (float)x[e] * c + (float)p[e] * sn : (float)x[e] * c - (float)p[e] * sn;
+          }
+        } else {
+#pragma unroll
+          for (int e = 0; e < VEC; ++e) y[r][e] = (float)x[e];
+        }
+#pragma unroll
+        for (int e = 0; e < VEC; ++e) ss += y[r][e] * y[r][e];
+      }
+    }
+    float inv = 1.0f;
+    if (unit_eps >= 0.f) inv = 1.0f / sqrtf(wave_sum(ss) / DK + unit_eps);
+#pragma unroll
+    for (int r = 0; r < kHalfRegs; ++r) {
+      const int i = (lane + 64 * r) * VEC;
+      if (i < DK) {
+        vec o;
+#pragma unroll
+        for (int e = 0; e < VEC; ++e) o[e] = (TA)(y[r][e] * inv);
+        *reinterpret_cast<vec*>(dst + i) = o;
+      }
+    }
+  }
+}
+
 constexpr int kMaxVChunks = 8;  // DV <= 512
 
 template <typename TA, bool SIG>
@@ -354,7 +452,7 @@ __global__ __launch_bounds__(256) void window_attention_kernel(
     TA* __restrict__ out, int ldo, int TH, int H, int G, int DK, int DV, float scale, float softcap, int window,
     const float* __restrict__ r1, const float* __restrict__ r2, const TA* __restrict__ gate, int ldg, int skip_len,
     const float* __restrict__ sig_bias, float out_scale, int nsplit, float* __restrict__ part, int chunk,
-    const float* __restrict__ hscale, int has_sink, float sink, const float* __restrict__ hsink) {
+    const float* __restrict__ hscale, int has_sink, float sink, const float* __restrict__ hsink, int ghead) {
   extern __shared__ float lds[];
   const int wid = threadIdx.x >> 6, lane = threadIdx.x & 63;
   const int th = blockIdx.x * 4 + wid;
@@ -458,7 +556,7 @@ __global__ __launch_bounds__(256) void window_attention_kernel(
     const int c = lane + 64 * n;
     if (c < DV) {
       float y = acc[n] * inv_l;
-      if (gate) y *= 1.0f / (1.0f + expf(-(float)gate[(size_t)t * ldg + (size_t)h * DV + c]));
+      if (gate) y *= 1.0f / (1.0f + expf(-(float)gate[(size_t)t * ldg + (ghead ? h : (size_t)h * DV + c)]));
       o[c] = (TA)y;
     }
   }
@@ -482,7 +580,7 @@ __global__ __launch_bounds__(256) void softmax_split_reduce_kernel(const float* 
                                                                    TA* __restrict__ out, int ldo, int T, int H, int DV,
                                                                    const TA* __restrict__ gate, int ldg, float out_scale,
                                                                    int has_sink, float sink,
-                                                                   const float* __restrict__ hsink) {
+                                                                   const float* __restrict__ hsink, int ghead) {
   const long e = (long)blockIdx.x * 256 + threadIdx.x;
   if (e >= (long)T * H * DV) return;
   const int th = (int)(e / DV), c = (int)(e % DV), t = th / H, h = th - t * H;
@@ -498,7 +596,7 @@ __global__ __launch_bounds__(256) void softmax_split_reduce_kernel(const float* 
     den = fmaf(p[DV + 1], f, den);
   }
   float y = num / den * out_scale;
-  if (gate) y *= 1.0f / (1.0f + expf(-(float)gate[(size_t)t * ldg + (size_t)h * DV + c]));
+  if (gate) y *= 1.0f / (1.0f + expf(-(float)gate[(size_t)t * ldg + (ghead ? h : (size_t)h * DV + c)]));
   out[(size_t)t * ldo + (size_t)h * DV + c] = (TA)y;
 }
 
@@ -540,7 +638,7 @@ __global__ __launch_bounds__(256) void window_attention_mfma_kernel(
     bf16* __restrict__ out, int ldo, int H, int G, float scale, float softcap, int window, const float* __restrict__ r1,
     const float* __restrict__ r2, const bf16* __restrict__ gate, int ldg, const float* __restrict__ sig_bias,
     float out_scale, int chunk, const float* __restrict__ hscale, int has_sink, float sink,
-    const float* __restrict__ hsink) {
+    const float* __restrict__ hsink, int ghead) {
   const int wid = threadIdx.x >> 6, lane = threadIdx.x & 63;
   const int h = blockIdx.y * 4 + wid;
   if (h >= H) return;
@@ -651,7 +749,8 @@ __global__ __launch_bounds__(256) void window_attention_mfma_kernel(
     inv_l /= l;
   }
   bf16* o = out + (size_t)t * ldo + (size_t)h * DV;
-  const bf16* gr = gate ? gate + (size_t)t * ldg + (size_t)h * DV : nullptr;
+  const bf16* gr = gate && !ghead ? gate + (size_t)t * ldg + (size_t)h * DV : nullptr;
+  if (gate && ghead) inv_l *= 1.0f / (1.0f + __expf(-(float)gate[(size_t)t * ldg + h]));
 #pragma unroll
   for (int i = 0; i < DV / 32; ++i) {
 #pragma unroll
@@ -674,17 +773,18 @@ void launch_window_mfma(const void* q, const void* k_cache, const void* v_cache,
                         const int* cu_q, const int* ctx, int S, void* out, int ldo, int T, int H, int G, float scale,
                         float softcap, int window, const float* r1, const float* r2, const void* gate, int ldg,
                         const float* sig_bias, int sig, float out_scale, hipStream_t st, int chunk, const float* hscale,
-                        int has_sink, float sink, const float* hsink) {
+                        int has_sink, float sink, const float* hsink, int ghead) {
   const dim3 grid((T + kTileQ - 1) / kTileQ + S, (H + 3) / 4);
   if (sig)
     window_attention_mfma_kernel<DK, DV, true><<<grid, 256, 0, st>>>(
         (const bf16*)q, (const bf16*)k_cache, (const bf16*)v_cache, block_tables, maxb, cu_q, ctx, S, (bf16*)out, ldo, H,
-        G, scale, softcap, window, r1, r2, (const bf16*)gate, ldg, sig_bias, out_scale, chunk, hscale, has_sink, sink, hsink);
+        G, scale, softcap, window, r1, r2, (const bf16*)gate, ldg, sig_bias, out_scale, chunk, hscale, has_sink, sink, hsink,
+        ghead);
   else
     window_attention_mfma_kernel<DK, DV, false><<<grid, 256, 0, st>>>(
         (const bf16*)q, (const bf16*)k_cache, (const bf16*)v_cache, block_tables, maxb, cu_q, ctx, S, (bf16*)out, ldo, H,
         G, scale, softcap, window, r1, r2, (const bf16*)gate, ldg, sig_bias, out_scale, chunk, hscale, has_sink, sink,
-        hsink);
+        hsink, ghead);
 }
 
 }  // namespace
@@ -769,6 +869,29 @@ void gai_rotary_kv_write(const void* q, int ldq, const void* k, int ldk, const v
   GAI_LAUNCH_CHECK();
 }
 
+void gai_rotary_half_kv_write(const void* q, int ldq, const void* k, int ldk, const void* v, int ldv, const int* positions,
+                              const int* slots, void* q_out, void* k_cache, void* v_cache, int T, int H, int G, int DK,
+                              int DV, const double* inv_freq, int half, float unit_eps, int dt, hipStream_t st) {
+  if (T == 0) return;
+  if (half < 0 || 2 * half > DK || DK > 64 * kHalfRegs)
+    gai_launch_error(__FILE__, __LINE__, "rotary_half_kv_write: rotated channels within a head of at most 512 channels");
+  const size_t lds = (size_t)(half > 0 ? 2 * half : 1) * sizeof(float);
+  const bool two = DK % 2 == 0 && half % 2 == 0 && ldq % 2 == 0 && ldk % 2 == 0 &&
+                   (((size_t)q | (size_t)k) & (dt ? 7 : 3)) == 0;
+  const bool tiles = T >= 64;   // v in tiles of 16 tokens
+  const int grid = T + (tiles ? (T + 15) / 16 : T);
+#define GAI_RH(TA, VEC_, VT_)                                                                                        \
+  rotary_half_kv_write_kernel<TA, VEC_, VT_><<<grid, 256, lds, st>>>((const TA*)q, ldq, (const TA*)k, ldk, (const TA*)v, ldv, \
+                                                                     positions, slots, (TA*)q_out, (TA*)k_cache,     \
+                                                                     (TA*)v_cache, T, H, G, DK, DV, inv_freq, half, unit_eps)
+#define GAI_RH2(TA, VEC_) if (tiles) GAI_RH(TA, VEC_, 16); else GAI_RH(TA, VEC_, 1)
+  if (dt) { if (two) { GAI_RH2(float, 2); } else { GAI_RH2(float, 1); } }
+  else { if (two) { GAI_RH2(bf16, 2); } else { GAI_RH2(bf16, 1); } }
+#undef GAI_RH2
+#undef GAI_RH
+  GAI_LAUNCH_CHECK();
+}
+
 // Key splits of a decode step (every row a single token): enough waves to give each SIMD a few
 int gai_sigmoid_attention_splits(int T, int S, int H) {
   if (T != S || T * H >= 2048) return 1;
@@ -780,7 +903,8 @@ void gai_window_attention(const void* q, const void* k_cache, const void* v_cach
                           const int* cu_q, const int* ctx, int S, void* out, int ldo, int T, int H, int G, int DK, int DV,
                           float scale, float softcap, int window, const float* r1, const float* r2, const void* gate,
                           int ldg, const float* sig_bias, int sig, float out_scale, int dt, hipStream_t st,
-                          float* part, int chunk, const float* hscale, int has_sink, float sink, const float* hsink) {
+                          float* part, int chunk, const float* hscale, int has_sink, float sink, const float* hsink,
+                          int ghead) {
   if (T == 0 || S == 0) return;
   if (hsink) has_sink = 1;
   if (sig && (chunk > 0 || hscale || has_sink))
@@ -797,7 +921,7 @@ void gai_window_attention(const void* q, const void* k_cache, const void* v_cach
   if (DK == K_ && DV == V_) {                                                                                        \
     launch_window_mfma<K_, V_>(q, k_cache, v_cache, block_tables, maxb, cu_q, ctx, S, out, ldo, T, H, G, scale,      \
                                softcap, window, r1, r2, gate, ldg, sig_bias, sig, out_scale, st, chunk, hscale,       \
-                               has_sink, sink, hsink);                                                               \
+                               has_sink, sink, hsink, ghead);                                                        \
     skip_len = kMfmaMinLen;                                                                                          \
   }
     GAI_WIN(64, 64) GAI_WIN(64, 128) GAI_WIN(128, 64) GAI_WIN(128, 128) GAI_WIN(256, 256)
@@ -811,7 +935,7 @@ void gai_window_attention(const void* q, const void* k_cache, const void* v_cach
   window_attention_kernel<TA, SIG_><<<dim3(grid, nsplit), 256, lds, st>>>(                                           \
       (const TA*)q, (const TA*)k_cache, (const TA*)v_cache, block_tables, maxb, cu_q, ctx, S, (TA*)out, ldo, TH, H, G, \
       DK, DV, scale, softcap, window, r1, r2, (const TA*)gate, ldg, skip_len, sig_bias, out_scale, nsplit, part,    \
-      chunk, hscale, has_sink, sink, hsink)
+      chunk, hscale, has_sink, sink, hsink, ghead)
   if (dt) {
     if (sig) GAI_ROW(float, true); else GAI_ROW(float, false);
   } else {
@@ -823,11 +947,11 @@ void gai_window_attention(const void* q, const void* k_cache, const void* v_cach
     if (dt)
       softmax_split_reduce_kernel<float><<<(unsigned)((n + 255) / 256), 256, 0, st>>>(part, nsplit, (float*)out, ldo, T, H,
                                                                                        DV, (const float*)gate, ldg,
-                                                                                       out_scale, has_sink, sink, hsink);
+                                                                                       out_scale, has_sink, sink, hsink, ghead);
     else
       softmax_split_reduce_kernel<bf16><<<(unsigned)((n + 255) / 256), 256, 0, st>>>(part, nsplit, (bf16*)out, ldo, T, H,
                                                                                       DV, (const bf16*)gate, ldg,
-                                                                                      out_scale, has_sink, sink, hsink);
+                                                                                      out_scale, has_sink, sink, hsink, ghead);
   } else if (nsplit > 1) {
     const long n = (long)T * H * DV;
     if (dt)

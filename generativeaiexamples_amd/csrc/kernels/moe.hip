@@ -40,10 +40,10 @@ constexpr int kMTile = MBM * MBK * 2;
 
 __global__ void moe_route_kernel(const float* __restrict__ logits, int T, int E, int k, int renorm,
                                  int* __restrict__ ids, float* __restrict__ w, int sigmoid,
-                                 const float* __restrict__ bias, float eps) {
+                                 const float* __restrict__ bias, float eps, int ld) {
   const int t = blockIdx.x * blockDim.x + threadIdx.x;
   if (t >= T) return;
-  const float* x = logits + (size_t)t * E;
+  const float* x = logits + (size_t)t * ld;
   float mx = -INFINITY;
   for (int e = 0; e < E; ++e) mx = fmaxf(mx, x[e]);
   float s = 0.f;
@@ -601,10 +601,10 @@ void gai_moe_dispatch(const int* ids, int n, int k, int E, int* a_rows, int* off
 }
 
 void gai_moe_route(const float* logits, int T, int E, int k, int renorm, int* ids, float* w, hipStream_t st,
-                   int sigmoid, const float* bias, float eps) {
+                   int sigmoid, const float* bias, float eps, int ld) {
   if (T == 0) return;
   if (k < 1 || k > 16 || k > E) gai_launch_error(__FILE__, __LINE__, "moe_route: 1 <= top-k <= min(16, experts)");
-  moe_route_kernel<<<(T + 255) / 256, 256, 0, st>>>(logits, T, E, k, renorm, ids, w, sigmoid, bias, eps);
+  moe_route_kernel<<<(T + 63) / 64, 64, 0, st>>>(logits, T, E, k, renorm, ids, w, sigmoid, bias, eps, ld ? ld : E);
   GAI_LAUNCH_CHECK();
 }
 

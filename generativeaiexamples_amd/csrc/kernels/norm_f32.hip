@@ -11,6 +11,8 @@
 //   gate_group_norm   g = y * silu(z);  out = g * rsqrt(mean_group(g^2) + eps) * w, the row cut into equal groups
 //   add_dyt_f32       res += delta (+ extra);  out = tanh(alpha * res) * w + b   (dynamic tanh: a norm without statistics,
 //                     so the pass is purely element-wise: four elements per thread, no reduction)
+//   parallel_add_norm res += sa * a + sb * b (per-channel scales);  h1 / h2 = rmsnorm(res) * w1 / w2: between two parallel
+//                     layers (mixer beside feed-forward, each with its own norm of the same sum), one workgroup per row
 //   act_mul           out = act(a) (* b), act: silu | squared ReLU | cap * tanh(a / cap) | tanh GELU, or the clamped gated
 //                     activation min(a, cap) * sigmoid(1.702 min(a, cap)) * (clamp(b, +-cap) + 1); fp32 arithmetic, a / b column
 //                     slices of wider rows, out bf16 or fp32
@@ -55,6 +57,79 @@ __global__ __launch_bounds__(256) void add_rmsnorm_f32_kernel(float* __restrict_
   s = wave_sum(s);
   const float inv = 1.0f / sqrtf(s / D + eps);
   for (int i = lane; i < D; i += 64) o[i] = (TA)(r[i] * inv * w[i]);
+}
+
+// One workgroup per row (as many threads as the row has groups of VEC channels, at most 256), the new sum kept in
+// registers between the passes (up to kParRegs groups per thread; what is past them is re-read).
+constexpr int kParRegs = 8;
+
+template <typename TA, int VEC>
+__global__ __launch_bounds__(256) void parallel_add_norm_kernel(float* __restrict__ res, const TA* __restrict__ a, int lda,
+                                                                const float* __restrict__ sa, const TA* __restrict__ b,
+                                                                int ldb, const float* __restrict__ sb,
+                                                                const float* __restrict__ w1, TA* __restrict__ h1,
+                                                                const float* __restrict__ w2, TA* __restrict__ h2, int D,
+                                                                float eps) {
+  typedef TA vec __attribute__((ext_vector_type(VEC)));
+  typedef float fvec __attribute__((ext_vector_type(VEC)));
+  __shared__ float scratch[16];
+  const int row = blockIdx.x, tid = threadIdx.x, step = blockDim.x * VEC;
+  float* r = res + (size_t)row * D;
+  const TA* ar = a ? a + (size_t)row * lda : nullptr;
+  const TA* br = b ? b + (size_t)row * ldb : nullptr;
+  auto sum = [&](int i) {
+    fvec x = *reinterpret_cast<const fvec*>(r + i);
+    if (ar) {
+      const vec y = *reinterpret_cast<const vec*>(ar + i);
+#pragma unroll
+      for (int e = 0; e < VEC; ++e) x[e] = fmaf(sa ? sa[i + e] : 1.0f, (float)y[e], x[e]);
+    }
+    if (br) {
+      const vec y = *reinterpret_cast<const vec*>(br + i);
+#pragma unroll
+      for (int e = 0; e < VEC; ++e) x[e] = fmaf(sb ? sb[i + e] : 1.0f, (float)y[e], x[e]);
+    }
+    if (ar || br) *reinterpret_cast<fvec*>(r + i) = x;
+    return x;
+  };
+  fvec v[kParRegs];
+  float s = 0.f;
+#pragma unroll
+  for (int q = 0; q < kParRegs; ++q) {
+    const int i = tid * VEC + step * q;
+    if (i < D) {
+      v[q] = sum(i);
+#pragma unroll
+      for (int e = 0; e < VEC; ++e) s = fmaf(v[q][e], v[q][e], s);
+    }
+  }
+  for (int i = tid * VEC + step * kParRegs; i < D; i += step) {
+    const fvec x = sum(i);
+#pragma unroll
+    for (int e = 0; e < VEC; ++e) s = fmaf(x[e], x[e], s);
+  }
+  if (!h1 && !h2) return;
+  s = block_sum(s, scratch);
+  const float inv = 1.0f / sqrtf(s / D + eps);
+  auto put = [&](const fvec& x, int i, const float* w, TA* h) {
+    vec o;
+#pragma unroll
+    for (int e = 0; e < VEC; ++e) o[e] = (TA)(x[e] * inv * w[i + e]);
+    *reinterpret_cast<vec*>(h + (size_t)row * D + i) = o;
+  };
+#pragma unroll
+  for (int q = 0; q < kParRegs; ++q) {
+    const int i = tid * VEC + step * q;
+    if (i < D) {
+      if (h1) put(v[q], i, w1, h1);
+      if (h2) put(v[q], i, w2, h2);
+    }
+  }
+  for (int i = tid * VEC + step * kParRegs; i < D; i += step) {
+    const fvec x = *reinterpret_cast<const fvec*>(r + i);
+    if (h1) put(x, i, w1, h1);
+    if (h2) put(x, i, w2, h2);
+  }
 }
 
 // Few rows (decode steps): one workgroup per row instead of one wave, the summed values kept in registers between the
@@ -588,5 +663,24 @@ void gai_act_mul(const void* a, int lda, const void* b, int ldb, void* out, int 
   else if (dt_out) GAI_AM(bf16, float);
   else GAI_AM(bf16, bf16);
 #undef GAI_AM
+  GAI_LAUNCH_CHECK();
+}
+
+// dt: a / b / h1 / h2 alike, 0 = bf16, 1 = fp32
+void gai_parallel_add_norm_f32(float* res, const void* a, int lda, const float* sa, const void* b, int ldb, const float* sb,
+                               const float* w1, void* h1, const float* w2, void* h2, int T, int D, float eps, int dt,
+                               hipStream_t st) {
+  if (T == 0 || D == 0) return;
+  if ((h1 && !w1) || (h2 && !w2)) gai_launch_error(__FILE__, __LINE__, "parallel_add_norm: every output has a norm weight");
+  const size_t mask = dt ? 15 : 7;
+  const bool four = D % 4 == 0 && (!a || lda % 4 == 0) && (!b || ldb % 4 == 0) && ((size_t)res & 15) == 0 &&
+                    (((size_t)a | (size_t)b | (size_t)h1 | (size_t)h2) & mask) == 0;
+  const int groups = four ? D / 4 : D, nt = groups >= 256 ? 256 : (groups + 63) / 64 * 64;
+#define GAI_PAN(TA, VEC_)                                                                                            \
+  parallel_add_norm_kernel<TA, VEC_><<<T, nt, 0, st>>>(res, (const TA*)a, lda, sa, (const TA*)b, ldb, sb, w1, (TA*)h1, w2, \
+                                                       (TA*)h2, D, eps)
+  if (dt) { if (four) GAI_PAN(float, 4); else GAI_PAN(float, 1); }
+  else { if (four) GAI_PAN(bf16, 4); else GAI_PAN(bf16, 1); }
+#undef GAI_PAN
   GAI_LAUNCH_CHECK();
 }
