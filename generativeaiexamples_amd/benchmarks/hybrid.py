@@ -1,4 +1,5 @@
 """Prefill and decode throughput of the hybrid decoders at layer sizes of real models (random weights), side by side:
+Bamanex (windowed grouped-query attention with sinks and head gates beside the feed-forward, dense and routed layers in turn),
 Luketar (full-context latent attention with sinks and an output gate, matrix-memory LSTM layers, four fp32 residual streams
 joined by hyper-connections, clamped gated experts plus a shared expert on every layer), Vipolix (gated linear attention layers and layers of chunk-local attention beside a generalised delta rule, token shift,
 group-routed clamped experts plus a gated shared expert on every layer, a per-layer token input; fp32 residual / state),
@@ -29,10 +30,10 @@ SIZES = {  # name: (width, layers, ff, heads, head_dim)
 
 def add_args(ap):
     ap.add_argument("--hybrid", action="store_true",
-                    help="prefill / decode throughput of Luketar, Vipolix, Lituvik, Ronavik, Pinavik and Qwen3-Next at equal layer sizes "
-                         "(one GPU)")
+                    help="prefill / decode throughput of Bamanex, Luketar, Vipolix, Lituvik, Ronavik, Pinavik and Qwen3-Next at "
+                         "equal layer sizes (one GPU)")
     ap.add_argument("--hybrid-sizes", default="1k,2k", help="comma list of " + ",".join(SIZES))
-    ap.add_argument("--hybrid-models", default="luketar,vipolix,lituvik,ronavik,pinavik,qwen3-next")
+    ap.add_argument("--hybrid-models", default="bamanex,luketar,vipolix,lituvik,ronavik,pinavik,qwen3-next")
     ap.add_argument("--hybrid-prefill", default="2048,8192", help="prompt lengths of the prefill measurement")
     ap.add_argument("--hybrid-decode", default="1,16,64", help="batch sizes of the decode measurement")
     ap.add_argument("--hybrid-context", type=int, default=1024)
@@ -41,6 +42,10 @@ def add_args(ap):
 
 def build(model: str, size: str, window: int, device):
     W, L, F, H, hd = SIZES[size]
+    if model == "bamanex":
+        from ..models.bamanex import BamanexConfig, BamanexModel
+
+        return BamanexModel(BamanexConfig.sized(W, L, F, H, hd, window=window, experts=8, top=2), device=device).random_init(0)
     if model == "luketar":
         from ..models.luketar import LuketarConfig, LuketarModel
 

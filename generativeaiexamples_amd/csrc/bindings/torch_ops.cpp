@@ -379,9 +379,9 @@ void sim_topk(const Tensor& Q, const Tensor& X, const Tensor& bias, int64_t n_ro
 
 void moe_route(const Tensor& logits, int64_t k, bool renorm, Tensor& ids, Tensor& w, bool sigmoid,
                const optional<Tensor>& bias, double eps) {
-  check_dev(logits, "router logits");  // rows may be a column slice of a wider projection
-  TORCH_CHECK(logits.scalar_type() == at::kFloat && logits.dim() == 2 && (logits.stride(1) == 1 || logits.size(1) == 1),
-              "moe_route: fp32 logits [T, E] with contiguous rows");
+  TORCH_CHECK(logits.is_cuda() && logits.scalar_type() == at::kFloat && logits.dim() == 2 &&
+                  (logits.stride(1) == 1 || logits.size(1) == 1),
+              "moe_route: fp32 GPU logits [T, E] with contiguous rows");  // a column slice of a wider projection
   check_i32(ids, "topk ids");
   check_f32(w, "topk weights");
   TORCH_CHECK(ids.is_contiguous() && w.is_contiguous() && ids.numel() == logits.size(0) * k && w.numel() == ids.numel(),
