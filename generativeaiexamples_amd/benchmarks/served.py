@@ -9,7 +9,7 @@ bench.py behind a ServiceHub, the same 1M-vector HBM index shard as the vector s
 ``--batch`` concurrent HTTP clients, released together, each streaming one ``/generate`` answer:
 
   client POST -> validation -> worker thread: query embed + exact scan, coalesced with the concurrent
-  queries (DynamicBatcher) on the high-priority retrieval stream -> rag prompt -> AsyncLLMEngine ->
+  queries (DynamicBatcher) on the retrieval stream -> rag prompt -> AsyncLLMEngine ->
   SSE frames awaited on the event loop -> client.
 
 The HTTP clients run in a separate process (``served_client``, spawned before the GPU is initialised),

@@ -93,7 +93,7 @@ class VectorStore:
     def _search_batch(self, items: List[Tuple[str, int, Optional[float]]]) -> List[List[Tuple[Document, float]]]:
         """[(query, k, threshold)] -> hits per query: one query-embedding micro-batch and one exact scan of
         the index for all of them (the scan streams the whole index once per batch, not once per query),
-        on the high-priority retrieval stream."""
+        on the retrieval stream."""
         from ..utils.streams import on_retrieval_stream
 
         with on_retrieval_stream(self.index.device):

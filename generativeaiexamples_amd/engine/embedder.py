@@ -159,7 +159,7 @@ class Embedder:
     # ---- coalesced serving path (/v1/embeddings, chain-server queries)
     @property
     def batcher(self) -> DynamicBatcher:
-        """Concurrent embed requests -> one encoder call per batch, on the high-priority retrieval stream."""
+        """Concurrent embed requests -> one encoder call per batch, on the retrieval stream."""
         if getattr(self, "_batcher", None) is None:
             with self.lock:
                 if getattr(self, "_batcher", None) is None:

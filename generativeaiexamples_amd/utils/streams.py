@@ -1,10 +1,10 @@
 """HIP streams of the serving process.
 
 The generator engine thread replays its decode graphs on the default stream. The query path (embedding
-micro-batches and exact index scans, issued from retrieval threads) runs on a separate HIGH-priority
-stream per device, so a new query's embed + scan kernels are scheduled beside a running decode graph
-instead of queueing behind it (a K-step decode run is ~65 ms at batch 64). Work on this stream is
-self-contained: its inputs are host data or persistent index buffers, and its results are read back
+micro-batches and exact index scans, issued from retrieval threads) runs on a separate stream per device
+(of default priority: work on streams of different priorities can hang), so a new query's embed + scan
+kernels run beside a decode graph instead of queueing behind it (a K-step decode run is ~65 ms at batch
+64). Work on this stream is self-contained: its inputs are host data or persistent index buffers, and its results are read back
 (``.cpu()``) on the same stream before any other thread uses them.
 """
 from __future__ import annotations
@@ -26,8 +26,7 @@ def retrieval_stream(device) -> "torch.cuda.Stream | None":
     with _lock:
         s = _streams.get(key)
         if s is None:
-            lo, hi = torch.cuda.Stream.priority_range()  # hi is the numerically smallest = highest priority
-            s = _streams[key] = torch.cuda.Stream(device=torch.device("cuda", key), priority=hi)
+            s = _streams[key] = torch.cuda.Stream(device=torch.device("cuda", key))
         return s
 
 
