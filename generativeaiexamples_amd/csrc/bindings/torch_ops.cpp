@@ -138,7 +138,7 @@ bool gemm_rope_kv(const Tensor& A, const Tensor& B, const optional<Tensor>& bias
 // would read address 0 on the device, so refuse it on the host.
 static void check_epi_operands(int64_t epi, const optional<Tensor>& bias, const optional<Tensor>& R,
                                const char* what) {
-  TORCH_CHECK(epi >= 0 && epi <= 7, what, ": unknown epilogue ", epi);
+  TORCH_CHECK((epi >= 0 && epi <= 7) || epi == 10, what, ": unknown epilogue ", epi);
   const bool needs_bias = epi == 1 || epi == 2 || epi == 5 || epi == 6 || epi == 7;
   const bool needs_res = epi == 3 || epi == 5;
   TORCH_CHECK(!needs_bias || bias.has_value(), what, ": epilogue ", epi, " needs a bias");
@@ -156,7 +156,8 @@ void gemm(const Tensor& A, const Tensor& B, Tensor& C, const optional<Tensor>& b
   TORCH_CHECK(B.size(1) == K, "gemm: K mismatch");
   const bool f32 = C.scalar_type() == at::kFloat;
   TORCH_CHECK(f32 || C.scalar_type() == at::kBFloat16, "gemm: C must be bf16 or fp32");
-  const int ldc = epi == 4 ? N / 2 : N;
+  const int ldc = epi == 4 || epi == 10 ? N / 2 : N;
+  TORCH_CHECK(epi != 10 || N % 32 == 0, "geglu: gated rows come in [gate16 | up16] blocks");
   TORCH_CHECK(C.numel() == (int64_t)M * ldc, "gemm: C has wrong size");
   check_epi_operands(epi, bias, R, "gemm");
   if (bias) check_bf16(*bias, "bias");
@@ -395,6 +396,20 @@ void moe_route(const Tensor& logits, int64_t k, bool renorm, Tensor& ids, Tensor
                 (int)logits.stride(0));
 }
 
+void moe_router(const Tensor& x, const Tensor& W, int64_t E, int64_t k, double eps, Tensor& ids, Tensor& w) {
+  check_i32(ids, "topk ids");
+  check_f32(w, "topk weights");
+  const bool f32 = x.scalar_type() == at::kFloat;
+  TORCH_CHECK(x.is_cuda() && W.is_cuda() && (f32 || x.scalar_type() == at::kBFloat16) && W.scalar_type() == x.scalar_type(),
+              "moe_router: bf16 or fp32 GPU rows and weights");
+  TORCH_CHECK(x.dim() == 2 && x.stride(1) == 1 && W.dim() == 2 && W.is_contiguous() && W.size(1) == x.size(1) &&
+                  W.size(0) >= E, "moe_router: x [T, D], W [>= E, D]");
+  TORCH_CHECK(ids.is_contiguous() && w.is_contiguous() && ids.numel() == x.size(0) * k && w.numel() == ids.numel(),
+              "moe_router: ids / w [T, k]");
+  gai_moe_router(x.data_ptr(), (int)x.stride(0), W.data_ptr(), x.size(0), x.size(1), (int)E, (int)k, (float)eps,
+                 ids.data_ptr<int>(), w.data_ptr<float>(), f32 ? 1 : 0, cur_stream());
+}
+
 void moe_scale_rows(const Tensor& h, const Tensor& pos, const Tensor& w, Tensor& out) {
   check_dev(h, "h");
   check_i32(pos, "pos");
@@ -449,7 +464,8 @@ void gemm_splitk(const Tensor& A, const Tensor& B, Tensor& C, const optional<Ten
   TORCH_CHECK(M <= 64 && gai_gemm_splitk_ks(M, N, K) > 0, "gemm_splitk: needs M <= 64 and K % 128 == 0");
   const bool f32 = C.scalar_type() == at::kFloat;
   TORCH_CHECK(f32 || C.scalar_type() == at::kBFloat16, "gemm_splitk: C must be bf16 or fp32");
-  const int ldc = epi == 4 ? N / 2 : N;
+  const int ldc = epi == 4 || epi == 10 ? N / 2 : N;
+  TORCH_CHECK(epi != 10 || N % 32 == 0, "geglu: gated rows come in [gate16 | up16] blocks");
   TORCH_CHECK(C.numel() == (int64_t)M * ldc, "gemm_splitk: C has wrong size");
   TORCH_CHECK(ws.scalar_type() == at::kFloat && ws.is_cuda() &&
                   (size_t)ws.numel() * 4 >= gai_gemm_splitk_ws_bytes(M, N, K), "gemm_splitk: workspace too small");
@@ -493,6 +509,7 @@ void gemm_fp8(const Tensor& A, const Tensor& B, const Tensor& sa, const Tensor& 
   TORCH_CHECK(f32 || C.scalar_type() == at::kBFloat16, "gemm_fp8: C must be bf16 or fp32");
   const int ldc = epi == 4 ? N / 2 : N;
   TORCH_CHECK(C.numel() == (int64_t)M * ldc, "gemm_fp8: C has wrong size");
+  TORCH_CHECK(epi <= 7, "gemm_fp8: unknown epilogue");
   check_epi_operands(epi, bias, R, "gemm_fp8");
   if (bias) check_bf16(*bias, "bias");
   if (R) {
@@ -1031,6 +1048,7 @@ PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
                     (int)down, (int)offset, (int)y.numel(), (float)gain, y.data_ptr<float>(), cur_stream());
   });
   m.def("moe_route", &moe_route);
+  m.def("moe_router", &moe_router);
   m.def("moe_scale_rows", &moe_scale_rows);
   m.def("moe_gemm", &moe_gemm);
   m.def("moe_route_chosen", &moe_route_chosen);

@@ -6,7 +6,15 @@ namespace gai {
 
 enum { EPI_NONE = 0, EPI_BIAS = 1, EPI_BIAS_GELU = 2, EPI_RESIDUAL = 3, EPI_SWIGLU = 4, EPI_BIAS_RESIDUAL = 5,
        EPI_BIAS_RELU = 6, EPI_BIAS_QUICKGELU = 7, EPI_RELU2 = 8,
-       EPI_CLAMP_GLU = 9 /* [gate16 | up16] rows: min(g, p) sigmoid(1.702 min(g, p)) (clamp(u, +-p) + 1) */ };
+       EPI_CLAMP_GLU = 9 /* [gate16 | up16] rows: min(g, p) sigmoid(1.702 min(g, p)) (clamp(u, +-p) + 1) */,
+       EPI_GEGLU = 10 /* [gate16 | up16] rows: gelu_tanh(g) u */ };
+
+// epilogues that turn [gate16 | up16] column pairs into one column
+constexpr bool epi_glu(int epi) { return epi == EPI_SWIGLU || epi == EPI_GEGLU; }
+template <int EPI>
+__device__ __forceinline__ float glu_act(float g, float u) {
+  return (EPI == EPI_GEGLU ? gelu_tanh(g) : silu(g)) * u;
+}
 
 __device__ __forceinline__ float quick_gelu(float x) { return x / (1.0f + __expf(-1.702f * x)); }
 

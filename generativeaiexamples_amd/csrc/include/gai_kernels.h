@@ -143,6 +143,8 @@ int gai_moe_gemm_dec2(const void* A, const int* a_rows, const void* W, void* C, 
 // sigmoid: scores sigmoid(logit) per expert instead of a softmax over the experts (weights = the chosen scores)
 void gai_moe_route(const float* logits, int T, int E, int k, int renorm, int* ids, float* w, hipStream_t st,
                    int sigmoid = 0, const float* bias = nullptr, float eps = 0.f, int ld = 0);  // ld: row stride (0: E)
+void gai_moe_router(const void* x, int ldx, const void* W, int T, int D, int E, int k, float eps, int* ids, float* w, int dt,
+                    hipStream_t st);
 // dt: 0 bf16 (MFMA tiles when K % 64 == 0), 1 fp32 (generic grouped kernel, true fp32)
 void gai_moe_gemm(const void* A, const int* a_rows, const void* W, void* C, const int* offs, int E, int rows_total,
                   int N, int K, int act, hipStream_t st, int dt = 0, float actp = 0.f);

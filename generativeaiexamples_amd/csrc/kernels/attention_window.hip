@@ -25,7 +25,7 @@
 //
 // rotary_half_kv_write: rotation of the channel pairs (i, i + half), i < half, of every q and k head by position *
 // inv_freq[i] (fp64 table; the angle is formed and reduced in fp64), then (unit_eps >= 0) every q and k head divided by its
-// root mean square, then q -> q_out and k, v -> their cache slots; one wave64 per head.
+// root mean square, then q -> q_out and k, v -> their cache slots; a power of two of lanes per head.
 //
 // headnorm_kv_write: RMS norm of every q head and every k head over its own DK channels (one weight vector of size DK
 // shared by the heads), optionally times a query temperature 1 + coef * ln(floor((p + 1) / every) + 1) of the token's
@@ -350,16 +350,17 @@ __global__ __launch_bounds__(256) void rotary_kv_write_kernel(const TI* __restri
   }
 }
 
-// Workgroups of the first nqk: q and k heads of one token, a wave per head (up to 64 NJ groups of VEC channels in
-// registers); the others: v of VT tokens, a thread per channel, so that tokens filling a whole page store its V^T row at once.
+// Workgroups 0 .. T - 1: q and k heads of one token, `lph` lanes (a power of two) per head with NJ groups of VEC channels
+// each, so a wave holds 64 / lph heads; the others: v of VT tokens, a thread per channel, so that tokens filling a whole page
+// store its V^T row at once.
 constexpr int kHalfRegs = 8;
 
-template <typename TA, int VEC, int VT>
+template <typename TA, int VEC, int NJ, int VT>
 __global__ __launch_bounds__(256) void rotary_half_kv_write_kernel(
     const TA* __restrict__ q, int ldq, const TA* __restrict__ k, int ldk, const TA* __restrict__ v, int ldv,
     const int* __restrict__ positions, const int* __restrict__ slots, TA* __restrict__ q_out, TA* __restrict__ k_cache,
     TA* __restrict__ v_cache, int T, int H, int G, int DK, int DV, const double* __restrict__ inv_freq, int half,
-    float unit_eps) {
+    float unit_eps, int lph) {
   const int tid = threadIdx.x;
   if ((int)blockIdx.x >= T) {
     const int t0 = ((int)blockIdx.x - T) * VT, n = min(VT, T - t0), NV = G * DV, s0 = slots[t0];
@@ -385,7 +386,7 @@ __global__ __launch_bounds__(256) void rotary_half_kv_write_kernel(
     return;
   }
   extern __shared__ float cs[];  // cos[half] | sin[half]
-  const int t = blockIdx.x, wid = tid >> 6, lane = tid & 63;
+  const int t = blockIdx.x, lane = tid & (lph - 1);
   const double pos = (double)positions[t];
   for (int i = tid; i < half; i += 256) {
     const double a = pos * inv_freq[i];
@@ -399,16 +400,16 @@ __global__ __launch_bounds__(256) void rotary_half_kv_write_kernel(
   const int slot = slots[t], off = slot & 15;
   const size_t page = slot >> 4;
   typedef TA vec __attribute__((ext_vector_type(VEC)));
-  for (int hh = wid; hh < H + G; hh += 4) {  // q heads, then k heads: wave-uniform
+  for (int hh = tid / lph; hh < H + G; hh += 256 / lph) {  // q heads, then k heads: uniform over the head's lanes
     const bool isq = hh < H;
     const int g = isq ? hh : hh - H;
     const TA* src = isq ? q + (size_t)t * ldq + (size_t)g * DK : k + (size_t)t * ldk + (size_t)g * DK;
     TA* dst = isq ? q_out + ((size_t)t * H + g) * DK : k_cache + ((page * G + g) * 16 + off) * DK;
-    float y[kHalfRegs][VEC];
+    float y[NJ][VEC];
     float ss = 0.f;
 #pragma unroll
-    for (int r = 0; r < kHalfRegs; ++r) {
-      const int i = (lane + 64 * r) * VEC;
+    for (int r = 0; r < NJ; ++r) {
+      const int i = (lane + lph * r) * VEC;
       if (i < DK) {
         const vec x = *reinterpret_cast<const vec*>(src + i);
         if (i < 2 * half) {   // VEC divides half: the group has one partner group
@@ -429,10 +430,13 @@ __global__ __launch_bounds__(256) void rotary_half_kv_write_kernel(
       }
     }
     float inv = 1.0f;
-    if (unit_eps >= 0.f) inv = 1.0f / sqrtf(wave_sum(ss) / DK + unit_eps);
+    if (unit_eps >= 0.f) {
+      for (int o = lph >> 1; o > 0; o >>= 1) ss += __shfl_xor(ss, o, 64);
+      inv = 1.0f / sqrtf(ss / DK + unit_eps);
+    }
 #pragma unroll
-    for (int r = 0; r < kHalfRegs; ++r) {
-      const int i = (lane + 64 * r) * VEC;
+    for (int r = 0; r < NJ; ++r) {
+      const int i = (lane + lph * r) * VEC;
       if (i < DK) {
         vec o;
 #pragma unroll
@@ -876,17 +880,22 @@ void gai_rotary_half_kv_write(const void* q, int ldq, const void* k, int ldk, co
   if (half < 0 || 2 * half > DK || DK > 64 * kHalfRegs)
     gai_launch_error(__FILE__, __LINE__, "rotary_half_kv_write: rotated channels within a head of at most 512 channels");
   const size_t lds = (size_t)(half > 0 ? 2 * half : 1) * sizeof(float);
-  const bool two = DK % 2 == 0 && half % 2 == 0 && ldq % 2 == 0 && ldk % 2 == 0 &&
-                   (((size_t)q | (size_t)k) & (dt ? 7 : 3)) == 0;
+  const auto on_grid = [&](int vec) {
+    return DK % vec == 0 && half % vec == 0 && ldq % vec == 0 && ldk % vec == 0 &&
+           (((size_t)q | (size_t)k | (size_t)q_out | (size_t)k_cache) & (vec * (dt ? 4 : 2) - 1)) == 0;
+  };
+  const int wide = dt ? 4 : 8, per = DK / wide;   // 16-byte groups, one per lane when a head is a power of two of them
+  const bool one = on_grid(wide) && per <= 64 && (per & (per - 1)) == 0;
+  const bool two = on_grid(2);
   const bool tiles = T >= 64;   // v in tiles of 16 tokens
   const int grid = T + (tiles ? (T + 15) / 16 : T);
-#define GAI_RH(TA, VEC_, VT_)                                                                                        \
-  rotary_half_kv_write_kernel<TA, VEC_, VT_><<<grid, 256, lds, st>>>((const TA*)q, ldq, (const TA*)k, ldk, (const TA*)v, ldv, \
-                                                                     positions, slots, (TA*)q_out, (TA*)k_cache,     \
-                                                                     (TA*)v_cache, T, H, G, DK, DV, inv_freq, half, unit_eps)
-#define GAI_RH2(TA, VEC_) if (tiles) GAI_RH(TA, VEC_, 16); else GAI_RH(TA, VEC_, 1)
-  if (dt) { if (two) { GAI_RH2(float, 2); } else { GAI_RH2(float, 1); } }
-  else { if (two) { GAI_RH2(bf16, 2); } else { GAI_RH2(bf16, 1); } }
+#define GAI_RH(TA, VEC_, NJ_, VT_)                                                                                   \
+  rotary_half_kv_write_kernel<TA, VEC_, NJ_, VT_><<<grid, 256, lds, st>>>(                                           \
+      (const TA*)q, ldq, (const TA*)k, ldk, (const TA*)v, ldv, positions, slots, (TA*)q_out, (TA*)k_cache, (TA*)v_cache, \
+      T, H, G, DK, DV, inv_freq, half, unit_eps, NJ_ == 1 ? per : 64)
+#define GAI_RH2(TA, VEC_, NJ_) if (tiles) GAI_RH(TA, VEC_, NJ_, 16); else GAI_RH(TA, VEC_, NJ_, 1)
+  if (dt) { if (one) { GAI_RH2(float, 4, 1); } else if (two) { GAI_RH2(float, 2, kHalfRegs); } else { GAI_RH2(float, 1, kHalfRegs); } }
+  else { if (one) { GAI_RH2(bf16, 8, 1); } else if (two) { GAI_RH2(bf16, 2, kHalfRegs); } else { GAI_RH2(bf16, 1, kHalfRegs); } }
 #undef GAI_RH2
 #undef GAI_RH
   GAI_LAUNCH_CHECK();

@@ -37,7 +37,7 @@ void gai_gemm(const void* A, const void* B, void* C, const void* bias, const voi
               int epi, int out_f32, int force, hipStream_t st, int bfrag) {
   if (M == 0 || N == 0) return;
   static_assert(EPI_NONE == 0 && EPI_BIAS == 1 && EPI_BIAS_GELU == 2 && EPI_RESIDUAL == 3 && EPI_SWIGLU == 4 &&
-                    EPI_BIAS_RESIDUAL == 5 && EPI_BIAS_RELU == 6 && EPI_BIAS_QUICKGELU == 7,
+                    EPI_BIAS_RESIDUAL == 5 && EPI_BIAS_RELU == 6 && EPI_BIAS_QUICKGELU == 7 && EPI_GEGLU == 10,
                 "gai_gemm_run<E> numbering");
   switch (epi) {
     case 0: return gai_gemm_run0(A, B, C, bias, R, M, N, K, ldc, out_f32, force, st, bfrag);
@@ -48,6 +48,7 @@ void gai_gemm(const void* A, const void* B, void* C, const void* bias, const voi
     case 5: return gai_gemm_run5(A, B, C, bias, R, M, N, K, ldc, out_f32, force, st, bfrag);
     case 6: return gai_gemm_run6(A, B, C, bias, R, M, N, K, ldc, out_f32, force, st, bfrag);
     case 7: return gai_gemm_run7(A, B, C, bias, R, M, N, K, ldc, out_f32, force, st, bfrag);
+    case 10: return gai_gemm_run10(A, B, C, bias, R, M, N, K, ldc, out_f32, force, st, bfrag);
     default:
       gai_launch_error(__FILE__, __LINE__, "gemm: unknown epilogue");
   }

@@ -223,7 +223,7 @@ __global__ __launch_bounds__(kThreads, 1) void gemm_dec2_kernel(const bf16* __re
       }
       dec_store8<true>(part, ((size_t)ks * M + m) * N + n, v);
     }
-  } else if (EPI == EPI_SWIGLU || EPI == EPI_CLAMP_GLU) {
+  } else if (epi_glu(EPI) || EPI == EPI_CLAMP_GLU) {
     // 16-column tiles (2j, 2j + 1) are (gate, up); output columns nb / 2 + 16 j + 8 h .. + 7
     constexpr int ITEMS = ROWS * NT;  // (m, j, h)
     for (int e = tid; e < ITEMS; e += kThreads) {
@@ -244,7 +244,7 @@ __global__ __launch_bounds__(kThreads, 1) void gemm_dec2_kernel(const bf16* __re
           up = fminf(fmaxf(up, -epi_param), epi_param);
           v[x] = g / (1.0f + expf(-1.702f * g)) * (up + 1.0f);
         } else {
-          v[x] = silu(g) * up;
+          v[x] = glu_act<EPI>(g, up);
         }
       }
       dec_store8<OUTF32>(C, (size_t)m * ldc + nb / 2 + 16 * j + 8 * h, v);
@@ -320,6 +320,15 @@ bool dec2_dispatch_epi(const void* A, const void* W, void* C, const void* bias, 
         return true;
       }
       return false;
+    case EPI_GEGLU:
+      if constexpr (NT >= 2) {
+        if (out_f32)
+          dec2_launch<MB, NT, EPI_GEGLU, true, false, PSW>(A, W, C, bias, R, M, N, K, ldc, st);
+        else
+          dec2_launch<MB, NT, EPI_GEGLU, false, false, PSW>(A, W, C, bias, R, M, N, K, ldc, st);
+        return true;
+      }
+      return false;
     default:
       return false;
   }
@@ -359,7 +368,7 @@ int dec2_pick_nt(int N, int K, bool swiglu) {
 template <int MB, bool PSW>
 bool dec2_run(const void* A, const void* W, void* C, const void* bias, const void* R, int M, int N, int K, int ldc,
               int epi, int out_f32, hipStream_t st) {
-  const int NT = dec2_pick_nt<MB>(N, K, epi == EPI_SWIGLU);
+  const int NT = dec2_pick_nt<MB>(N, K, epi_glu(epi));
   switch (NT) {
     case 8: return dec2_dispatch_epi<MB, 8, PSW>(A, W, C, bias, R, M, N, K, ldc, epi, out_f32, st);
     case 4: return dec2_dispatch_epi<MB, 4, PSW>(A, W, C, bias, R, M, N, K, ldc, epi, out_f32, st);
@@ -382,10 +391,10 @@ int gai_gemm_dec2_ok(int M, int N, int K, int epi) {
   // here (profiles/r5/config3_dec2_ab) - those keep the split-K kernels.
   static const int min_n = getenv("GAI_DEC2_MINN") ? atoi(getenv("GAI_DEC2_MINN")) : 16384;
   const bool shallow_shard = N >= 8192 && K <= 4096 && !getenv("GAI_DEC2_MINN");
-  if (M < 1 || M > 64 || N % 16 || (N < min_n && !shallow_shard) || (epi == EPI_SWIGLU && N % 32)) return 0;
+  if (M < 1 || M > 64 || N % 16 || (N < min_n && !shallow_shard) || (epi_glu(epi) && N % 32)) return 0;
   static const bool off = getenv("GAI_DEC2") && atoi(getenv("GAI_DEC2")) == 0;
   if (off) return 0;
-  const bool sw = epi == EPI_SWIGLU;
+  const bool sw = epi_glu(epi);
   if (M <= 16) return dec2_pick_nt<1>(N, K, sw) > 0;
   if (M <= 32) return dec2_pick_nt<2>(N, K, sw) > 0;
   return dec2_pick_nt<4>(N, K, sw) > 0;

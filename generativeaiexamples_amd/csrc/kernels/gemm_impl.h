@@ -138,7 +138,7 @@ __global__ __launch_bounds__(256, 2) void gemm_tiled_kernel(const bf16* __restri
   }
 
   // epilogue: lane holds D[m = 4(lane>>4)+r][n = lane&15] of each 16x16 tile
-  if (EPI == EPI_SWIGLU) {
+  if (epi_glu(EPI)) {
 #pragma unroll
     for (int i = 0; i < 4; ++i)
 #pragma unroll
@@ -150,7 +150,7 @@ __global__ __launch_bounds__(256, 2) void gemm_tiled_kernel(const bf16* __restri
           const int m = m0 + wm * 64 + 16 * i + 4 * (lane >> 4) + r;
           if (m >= M) continue;
           const float g = acc[i][2 * jp][r], u = acc[i][2 * jp + 1][r];
-          store_out<EPI_NONE, OUTF32>(C, nullptr, nullptr, ldc, m, nout, silu(g) * u);
+          store_out<EPI_NONE, OUTF32>(C, nullptr, nullptr, ldc, m, nout, glu_act<EPI>(g, u));
         }
       }
   } else {
@@ -253,15 +253,15 @@ __device__ __forceinline__ void epilogue_rows(const f32x4 (&acc_i)[NJ], void* C,
     }
     return;
   }
-  if (EPI == EPI_SWIGLU) {
+  if (epi_glu(EPI)) {
     // tiles (2jp, 2jp+1) = (gate, up) of output columns nb/2 + 16jp + 4q + r; pair jp = 2t, 2t+1
 #pragma unroll
     for (int t = 0; t < NJ / 4; ++t) {
       float h0[4], h1[4];
 #pragma unroll
       for (int r = 0; r < 4; ++r) {
-        h0[r] = silu(acc_i[4 * t][r]) * acc_i[4 * t + 1][r];
-        h1[r] = silu(acc_i[4 * t + 2][r]) * acc_i[4 * t + 3][r];
+        h0[r] = glu_act<EPI>(acc_i[4 * t][r], acc_i[4 * t + 1][r]);
+        h1[r] = glu_act<EPI>(acc_i[4 * t + 2][r], acc_i[4 * t + 3][r]);
         swap16(h0[r], h1[r]);
       }
       const int n = nb / 2 + 32 * t + 16 * (q & 1) + 8 * (q >> 1);
@@ -1230,7 +1230,7 @@ __global__ __launch_bounds__(512) void gemm_skinny_kernel(const bf16* __restrict
   __syncthreads();
 
   // element (m, n): i = m>>4, r = m&3, lane = ((m&15)>>2)*16 + (n&15), f = n>>4
-  if (EPI == EPI_SWIGLU) {
+  if (epi_glu(EPI)) {
     constexpr int NO = NB / 2;
     for (int e = tid; e < M * NO; e += 512) {
       const int m = e / NO, no = e % NO;
@@ -1243,7 +1243,7 @@ __global__ __launch_bounds__(512) void gemm_skinny_kernel(const bf16* __restrict
         u += part[(((w * MT + i) * NF + 2 * fp + 1) * 4 + r) * 64 + l];
       }
       const int nout = n0 / 2 + no;
-      if (2 * nout < N) store_out<EPI_NONE, OUTF32>(C, nullptr, nullptr, ldc, m, nout, silu(g) * u);
+      if (2 * nout < N) store_out<EPI_NONE, OUTF32>(C, nullptr, nullptr, ldc, m, nout, glu_act<EPI>(g, u));
     }
   } else {
     for (int e = tid; e < M * NB; e += 512) {
@@ -1502,9 +1502,9 @@ void launch_gemm(const void* A, const void* B, void* C, const void* bias, const 
   if (use_skinny) {
     if (!skinny_ok) gai_launch_error(__FILE__, __LINE__, "gemm_skinny: needs M<=128 and K%256==0");
     // two 16-row fragments per wave when there are enough column blocks to fill the chip
-    if (EPI != EPI_SWIGLU && N / 32 >= 512)
+    if (!epi_glu(EPI) && N / 32 >= 512)
       return launch_skinny_nf<2, EPI, OUTF32>(A, B, C, bias, R, M, N, K, ldc, st, bfrag);
-    if (EPI == EPI_SWIGLU) return launch_skinny_nf<2, EPI, OUTF32>(A, B, C, bias, R, M, N, K, ldc, st, bfrag);
+    if (epi_glu(EPI)) return launch_skinny_nf<2, EPI, OUTF32>(A, B, C, bias, R, M, N, K, ldc, st, bfrag);
     return launch_skinny_nf<1, EPI, OUTF32>(A, B, C, bias, R, M, N, K, ldc, st, bfrag);
   }
   if (K % TBK) gai_launch_error(__FILE__, __LINE__, "gemm_tiled: K must be a multiple of 64");
@@ -1559,3 +1559,4 @@ void gai_gemm_run4(GAI_GEMM_RUN_ARGS);
 void gai_gemm_run5(GAI_GEMM_RUN_ARGS);
 void gai_gemm_run6(GAI_GEMM_RUN_ARGS);
 void gai_gemm_run7(GAI_GEMM_RUN_ARGS);
+void gai_gemm_run10(GAI_GEMM_RUN_ARGS);

@@ -344,7 +344,7 @@ __global__ __launch_bounds__(256, 2) void gemm_dec_kernel(const bf16* __restrict
       }
       continue;
     }
-    if (EPI == EPI_SWIGLU) {
+    if (epi_glu(EPI)) {
       // columns [g16 u16 g16 u16]: the gate lanes (q even) pull the up half from the next group
       if (q & 1) continue;
       const float* up = tile + m * kLdsRow + 16 * (q + 1);
@@ -360,14 +360,14 @@ __global__ __launch_bounds__(256, 2) void gemm_dec_kernel(const bf16* __restrict
         bf16x8 o0, o1;
 #pragma unroll
         for (int c = 0; c < 8; ++c) {
-          o0[c] = (bf16)(silu(v[c]) * u[c]);
-          o1[c] = (bf16)(silu(v[8 + c]) * u[8 + c]);
+          o0[c] = (bf16)(glu_act<EPI>(v[c], u[c]));
+          o1[c] = (bf16)(glu_act<EPI>(v[8 + c], u[8 + c]));
         }
         store8(reinterpret_cast<bf16*>(C) + (size_t)m * ldc + oc, o0);
         store8(reinterpret_cast<bf16*>(C) + (size_t)m * ldc + oc + 8, o1);
       } else {
         for (int c = 0; c < 16; ++c)
-          if (n0 + 16 * q + 16 + c < N) store_out<EPI_NONE, OUTF32>(C, nullptr, nullptr, ldc, m, oc + c, silu(v[c]) * u[c]);
+          if (n0 + 16 * q + 16 + c < N) store_out<EPI_NONE, OUTF32>(C, nullptr, nullptr, ldc, m, oc + c, glu_act<EPI>(v[c], u[c]));
       }
     } else {
 #pragma unroll
@@ -441,16 +441,16 @@ __device__ __forceinline__ void sum_slabs_any(const float* p, size_t stride, int
 template <int EPI, bool OUTF32>
 __global__ __launch_bounds__(256) void splitk_reduce_kernel(const float* __restrict__ part, int KS, int M, int N,
                                                             void* C, const bf16* bias, const bf16* R, int ldc) {
-  const int ncol = EPI == EPI_SWIGLU ? N / 2 : N;
+  const int ncol = epi_glu(EPI) ? N / 2 : N;
   const long e = (long)blockIdx.x * 256 + threadIdx.x;
   if (e >= (long)M * ncol) return;
   const int m = (int)(e / ncol), j = (int)(e % ncol);
-  if (EPI == EPI_SWIGLU) {
+  if (epi_glu(EPI)) {
     const int g = (j >> 4) * 32 + (j & 15);  // interleaved per 16: [gate16 | up16]
     float vg[1] = {0.f}, vu[1] = {0.f};
     sum_slabs<1>(part + (size_t)m * N + g, (size_t)M * N, KS, vg);
     sum_slabs<1>(part + (size_t)m * N + g + 16, (size_t)M * N, KS, vu);
-    store_out<EPI_NONE, OUTF32>(C, nullptr, nullptr, ldc, m, j, silu(vg[0]) * vu[0]);
+    store_out<EPI_NONE, OUTF32>(C, nullptr, nullptr, ldc, m, j, glu_act<EPI>(vg[0], vu[0]));
   } else {
     float v[1] = {0.f};
     sum_slabs<1>(part + (size_t)m * N + j, (size_t)M * N, KS, v);
@@ -461,7 +461,7 @@ __global__ __launch_bounds__(256) void splitk_reduce_kernel(const float* __restr
 template <int EPI, bool OUTF32>
 void launch_reduce(const float* part, int KS, int M, int N, void* C, const void* bias, const void* R, int ldc,
                    hipStream_t st) {
-  const int ncol = EPI == EPI_SWIGLU ? N / 2 : N;
+  const int ncol = epi_glu(EPI) ? N / 2 : N;
   const long total = (long)M * ncol;
   splitk_reduce_kernel<EPI, OUTF32><<<(unsigned)((total + 255) / 256), 256, 0, st>>>(
       part, KS, M, N, C, (const bf16*)bias, (const bf16*)R, ldc);
@@ -571,6 +571,7 @@ void dispatch_stream_ks1(const void* A, const void* B, void* C, const void* bias
     GAI_SS(EPI_BIAS_GELU)
     GAI_SS(EPI_RESIDUAL)
     GAI_SS(EPI_SWIGLU)
+    GAI_SS(EPI_GEGLU)
     GAI_SS(EPI_BIAS_RESIDUAL)
     GAI_SS(EPI_BIAS_RELU)
     GAI_SS(EPI_BIAS_QUICKGELU)
@@ -958,6 +959,7 @@ void gai_gemm_splitk(const void* A, const void* B, void* C, const void* bias, co
     GAI_SKR(EPI_BIAS_GELU)
     GAI_SKR(EPI_RESIDUAL)
     GAI_SKR(EPI_SWIGLU)
+    GAI_SKR(EPI_GEGLU)
     GAI_SKR(EPI_BIAS_RESIDUAL)
     GAI_SKR(EPI_BIAS_RELU)
     GAI_SKR(EPI_BIAS_QUICKGELU)

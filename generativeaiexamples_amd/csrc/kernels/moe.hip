@@ -24,6 +24,7 @@
 //              top-2 choice scores added up); weights = the chosen plain scores renormalised (+ eps), scaled.
 // moe_route (chosen): bias is part of the logits; the top-k logits + bias are chosen and weighted by the softmax over the
 //              chosen ones only; libm expf, all fp32.
+// moe_router:  router product + softmax + top-k of decode-sized steps in one launch, a workgroup per token.
 // moe_gemm (clamped gated): g = min(gate, p), u = clamp(up, +-p), g sigmoid(1.702 g) (u + 1) on [gate16 | up16] rows.
 // moe_combine (residual gate): the residual row (a shared expert's output) times sigmoid of a per-token logit.
 // moe_scale_rows: expert-sorted copies of the token rows, each times its routing weight (experts whose routing weight
@@ -80,6 +81,73 @@ __global__ void moe_route_kernel(const float* __restrict__ logits, int T, int E,
   for (int j = 0; j < k; ++j) {
     ids[(size_t)t * k + j] = bi[j];
     w[(size_t)t * k + j] = (renorm && !sigmoid) ? bv[j] / tot : bv[j];
+  }
+}
+
+// Decode-sized steps: router product, softmax and top-k of a token in one workgroup (logits and scores stay in LDS). The
+// waves deal the experts out and dot them in fp32; wave 0 normalises and picks k times the largest score (the lower id wins
+// a tie); weights = chosen scores / (their sum + eps).
+template <typename TA, int VEC>
+__global__ __launch_bounds__(256) void moe_router_kernel(const TA* __restrict__ x, int ldx, const TA* __restrict__ W, int D,
+                                                         int E, int k, float eps, int* __restrict__ ids,
+                                                         float* __restrict__ w) {
+  typedef TA vec __attribute__((ext_vector_type(VEC)));
+  extern __shared__ float score[];  // [E]
+  const int t = blockIdx.x, wid = threadIdx.x >> 6, lane = threadIdx.x & 63;
+  const TA* xr = x + (size_t)t * ldx;
+  for (int e = wid; e < E; e += 4) {
+    const TA* wr = W + (size_t)e * D;
+    float a = 0.f;
+#pragma unroll 4
+    for (int i = lane * VEC; i < D; i += 64 * VEC) {
+      const vec p = *reinterpret_cast<const vec*>(xr + i), q = *reinterpret_cast<const vec*>(wr + i);
+#pragma unroll
+      for (int z = 0; z < VEC; ++z) a = fmaf((float)p[z], (float)q[z], a);
+    }
+    a = wave_sum(a);
+    if (lane == 0) score[e] = a;
+  }
+  __syncthreads();
+  if (wid) return;
+  float m = -INFINITY, s = 0.f;
+  for (int e = lane; e < E; e += 64) m = fmaxf(m, score[e]);
+  m = wave_max(m);
+  for (int e = lane; e < E; e += 64) {   // every lane touches only its own entries of the list
+    const float p = expf(score[e] - m);
+    score[e] = p;
+    s += p;
+  }
+  s = wave_sum(s);
+  for (int e = lane; e < E; e += 64) score[e] /= s;
+  float tot = eps, mine = 0.f;
+  int mid = 0;
+  for (int j = 0; j < k; ++j) {
+    float b = -1.f;
+    int id = E;
+    for (int e = lane; e < E; e += 64)
+      if (score[e] > b) {
+        b = score[e];
+        id = e;
+      }
+#pragma unroll
+    for (int o = 32; o > 0; o >>= 1) {
+      const float ob = __shfl_xor(b, o, 64);
+      const int oi = __shfl_xor(id, o, 64);
+      if (ob > b || (ob == b && oi < id)) {
+        b = ob;
+        id = oi;
+      }
+    }
+    if ((id & 63) == lane) score[id] = -2.f;   // taken
+    tot += b;
+    if (lane == j) {
+      mine = b;
+      mid = id;
+    }
+  }
+  if (lane < k) {
+    ids[(size_t)t * k + lane] = mid;
+    w[(size_t)t * k + lane] = mine / tot;
   }
 }
 
@@ -605,6 +673,22 @@ void gai_moe_route(const float* logits, int T, int E, int k, int renorm, int* id
   if (T == 0) return;
   if (k < 1 || k > 16 || k > E) gai_launch_error(__FILE__, __LINE__, "moe_route: 1 <= top-k <= min(16, experts)");
   moe_route_kernel<<<(T + 63) / 64, 64, 0, st>>>(logits, T, E, k, renorm, ids, w, sigmoid, bias, eps, ld ? ld : E);
+  GAI_LAUNCH_CHECK();
+}
+
+// dt: x / W 0 bf16, 1 fp32
+void gai_moe_router(const void* x, int ldx, const void* W, int T, int D, int E, int k, float eps, int* ids, float* w, int dt,
+                    hipStream_t st) {
+  if (T == 0) return;
+  if (E < 1 || E > 4096 || k < 1 || k > 16 || k > E)
+    gai_launch_error(__FILE__, __LINE__, "moe_router: 1 <= top-k <= min(16, experts), experts <= 4096");
+  const int wide = dt ? 4 : 8;
+  const bool ok = D % wide == 0 && ldx % wide == 0 && (((size_t)x | (size_t)W) & 15) == 0;
+  const size_t lds = E * sizeof(float);
+#define GAI_MR(TA, VEC_) moe_router_kernel<TA, VEC_><<<T, 256, lds, st>>>((const TA*)x, ldx, (const TA*)W, D, E, k, eps, ids, w)
+  if (dt) { if (ok) GAI_MR(float, 4); else GAI_MR(float, 1); }
+  else { if (ok) GAI_MR(bf16, 8); else GAI_MR(bf16, 1); }
+#undef GAI_MR
   GAI_LAUNCH_CHECK();
 }
 

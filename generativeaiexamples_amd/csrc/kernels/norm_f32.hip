@@ -258,26 +258,30 @@ __global__ __launch_bounds__(256) void head_norm_gate_kernel(const float* __rest
   }
 }
 
-template <typename TA>
+// blockIdx.y: 256 VEC columns of a row
+template <typename TA, int VEC>
 __global__ __launch_bounds__(256) void embed_scale_f32_kernel(const int* __restrict__ ids, const TA* __restrict__ table,
-                                                              float scale, float* __restrict__ out, int T, int D,
-                                                              int V, const int* __restrict__ positions,
+                                                              float scale, float* __restrict__ out, int D, int V,
+                                                              const int* __restrict__ positions,
                                                               const TA* __restrict__ pos_table, int P) {
-  const int lane = threadIdx.x & 63;
-  const int row = blockIdx.x * 4 + (threadIdx.x >> 6);
-  if (row >= T) return;
+  typedef TA vec __attribute__((ext_vector_type(VEC)));
+  typedef float fvec __attribute__((ext_vector_type(VEC)));
+  const int row = blockIdx.x, i = (blockIdx.y * 256 + threadIdx.x) * VEC;
+  if (i >= D) return;
   int id = ids[row];
   id = id < 0 ? 0 : (id >= V ? V - 1 : id);
-  const TA* e = table + (size_t)id * D;
-  float* o = out + (size_t)row * D;
+  const vec e = *reinterpret_cast<const vec*>(table + (size_t)id * D + i);
+  fvec o;
+#pragma unroll
+  for (int q = 0; q < VEC; ++q) o[q] = (float)e[q] * scale;
   if (pos_table) {
     int p = positions[row];
     p = p < 0 ? 0 : (p >= P ? P - 1 : p);
-    const TA* pe = pos_table + (size_t)p * D;
-    for (int i = lane; i < D; i += 64) o[i] = (float)e[i] * scale + (float)pe[i];
-  } else {
-    for (int i = lane; i < D; i += 64) o[i] = (float)e[i] * scale;
+    const vec pe = *reinterpret_cast<const vec*>(pos_table + (size_t)p * D + i);
+#pragma unroll
+    for (int q = 0; q < VEC; ++q) o[q] += (float)pe[q];
   }
+  *reinterpret_cast<fvec*>(out + (size_t)row * D + i) = o;
 }
 
 template <typename TY, typename TG, typename TA>
@@ -567,13 +571,13 @@ void gai_head_norm_gate(const float* o, const void* gate, int ldg, const float* 
 void gai_embed_scale_f32(const int* ids, const void* table, float scale, float* out, int T, int D, int V, int dt,
                          hipStream_t st, const int* positions, const void* pos_table, int P) {
   if (T == 0) return;
-  const int grid = (T + 3) / 4;
-  if (dt)
-    embed_scale_f32_kernel<float><<<grid, 256, 0, st>>>(ids, (const float*)table, scale, out, T, D, V, positions,
-                                                        (const float*)pos_table, P);
-  else
-    embed_scale_f32_kernel<bf16><<<grid, 256, 0, st>>>(ids, (const bf16*)table, scale, out, T, D, V, positions,
-                                                       (const bf16*)pos_table, P);
+#define GAI_EMB(TA, VEC_)                                                                                            \
+  embed_scale_f32_kernel<TA, VEC_><<<dim3(T, (D + 256 * VEC_ - 1) / (256 * VEC_)), 256, 0, st>>>(                    \
+      ids, (const TA*)table, scale, out, D, V, positions, (const TA*)pos_table, P)
+  const bool four = D % 4 == 0 && ((size_t)out & 15) == 0 && (((size_t)table | (size_t)pos_table) & (dt ? 15 : 7)) == 0;
+  if (dt) { if (four) GAI_EMB(float, 4); else GAI_EMB(float, 1); }
+  else { if (four) GAI_EMB(bf16, 4); else GAI_EMB(bf16, 1); }
+#undef GAI_EMB
   GAI_LAUNCH_CHECK();
 }
 

@@ -228,11 +228,13 @@ class BamanexModel(HybridDecoderBase):
         w["embed"], w["head"] = mat(sd["embed"]), mat(pad_rows(sd["head"], 16))   # padded logits are cut off by forward()
         w["final.norm"] = f32((1 + sd["final.norm"].float()) * c.logit_scale)
 
-        def gated(src, dst, extra=()):
-            # wide feed-forwards padded with zeros to the split-K decode GEMM's grid
+        def gated(src, dst, fused, extra=()):
+            # wide feed-forwards padded with zeros to the split-K decode GEMM's grid; fused: rows interleaved for the gated
+            # epilogue of the GEMM
             wide = 512 if bf and sd[src + "gate"].shape[0] >= 1024 else 16
-            rows = [pad_rows(sd[src + "gate"], wide), pad_rows(sd[src + "up"], wide)]
-            w[dst + "in"] = mat(pad_rows(torch.cat(rows + [sd[e].float().reshape(1, -1) for e in extra]), 16))
+            gate, up = pad_rows(sd[src + "gate"], wide), pad_rows(sd[src + "up"], wide)
+            rows = torch.cat([gate, up] + [sd[e].float().reshape(1, -1) for e in extra])
+            w[dst + "in"] = mat(ops.interleave_gate_up(gate, up) if fused else pad_rows(rows, 16))
             w[dst + "down"] = mat(pad_rows(sd[src + "down"].t(), wide).t())
 
         for i, l in enumerate(c.layers):
@@ -248,13 +250,13 @@ class BamanexModel(HybridDecoderBase):
                 continue
             w[p + "norm2"], w[p + "ls2"] = f32(1 + sd[p + "norm2"].float()), f32(sd[p + "ls2"])
             if ml["kind"] == "dense":
-                gated(q, q)
+                gated(q, q, bf)
                 continue
             w[q + "router"] = mat(pad_rows(sd[q + "router"], 16))
             gate_up, down = stack_gated_experts(sd, q, ml["router"]["experts"], 64 if bf else 16)
             w[q + "gate_up"], w[q + "e.down"] = mat(gate_up), mat(down)
             if ml.get("shared"):
-                gated(q + "shared.", q + "shared.", (q + "shared.sg",))
+                gated(q + "shared.", q + "shared.", False, (q + "shared.sg",))
         return self
 
     def random_init(self, seed: int = 0):
@@ -274,28 +276,33 @@ class BamanexModel(HybridDecoderBase):
                                    window=m["window"], sink=w[x + "sink"], gate=proj[:, c:c + H])
         return ops.linear(att, w[x + "o"], w[x + "o.b"])
 
-    def _gated(self, h, p, act, limit=0.0):
-        """W_down of the gated activation of one fused gate | up projection -> (output, the projection's columns past
-        gate | up)."""
-        w_down = self.w[p + "down"]
-        F_ = w_down.shape[1]
-        gu = ops.linear(h, self.w[p + "in"])
-        mid = ops.act_mul(gu[:, :F_], gu[:, F_:2 * F_], act, self.dtype, cap=float(limit))
-        return ops.linear(mid, w_down), gu[:, 2 * F_:]
+    def _dense(self, h, p):
+        w, F_ = self.w, self.w[p + "down"].shape[1]
+        if self.dtype == torch.bfloat16:   # gate / up rows interleaved: the activation is the GEMM's epilogue
+            mid = ops.linear(h, w[p + "in"], act="geglu")
+        else:
+            gu = ops.linear(h, w[p + "in"])
+            mid = ops.act_mul(gu[:, :F_], gu[:, F_:], "gelu_tanh", self.dtype)
+        return ops.linear(mid, w[p + "down"])
+
+    def _shared(self, h, p, limit):
+        """Shared expert -> (output, its gate logit per token): one fused gate | up | sg projection."""
+        w, F_ = self.w, self.w[p + "down"].shape[1]
+        gu = ops.linear(h, w[p + "in"])
+        mid = ops.act_mul(gu[:, :F_], gu[:, F_:2 * F_], "clamp_glu", self.dtype, cap=float(limit))
+        return ops.linear(mid, w[p + "down"]), gu[:, 2 * F_:2 * F_ + 1]
 
     def _moe(self, h, ml, q):
         w, r = self.w, ml["router"]
-        E, top = r["experts"], r["top"]
-        logits = ops.linear(h, w[q + "router"], out_dtype=torch.float32)[:, :E]
-        ids, wts = ops.moe_route(logits, top, eps=ROUTE_EPS)
+        E, n = r["experts"], h.shape[0] * r["top"]
         shared = sgate = None
         if ml.get("shared"):
-            shared, rest = self._gated(h, q + "shared.", "clamp_glu", ml["shared"]["limit"])
-            sgate = rest[:, :1]
+            shared, sgate = self._shared(h, q + "shared.", ml["shared"]["limit"])
+        ids, wts = ops.moe_router(h, w[q + "router"], E, r["top"], ROUTE_EPS)
         rows, offs, pos = ops.moe_dispatch(ids, E)
-        n = h.shape[0] * top
         mid = ops.moe_gemm(h, rows, w[q + "gate_up"], offs, n, act="clamp_glu", act_param=float(ml["expert"]["limit"]))
-        return ops.moe_combine(ops.moe_gemm(mid, None, w[q + "e.down"], offs, n), pos, wts, shared, residual_gate=sgate)
+        out = ops.moe_gemm(mid, None, w[q + "e.down"], offs, n)
+        return ops.moe_combine(out, pos, wts, shared, residual_gate=sgate)
 
     # ------------------------------------------------------------------ forward
     def forward(self, fb: ForwardBatch, kv, decode_ws=None) -> torch.Tensor:
@@ -315,7 +322,7 @@ class BamanexModel(HybridDecoderBase):
             a, s1 = self._attention(h1, i, (i, t), fb, kv, seq), w[p + "ls1"]
             b = s2 = None
             if ml is not None:
-                b = self._moe(h2, ml, p + "mlp.") if ml["kind"] == "moe" else self._gated(h2, p + "mlp.", "gelu_tanh")[0]
+                b = self._moe(h2, ml, p + "mlp.") if ml["kind"] == "moe" else self._dense(h2, p + "mlp.")
                 s2 = w[p + "ls2"]
             if self.capture_residuals is not None:
                 ops.parallel_add_norm_f32(res, a, s1, b, s2)

@@ -55,7 +55,7 @@ def native_available() -> bool:
         return False
 
 
-EPI = {None: 0, "bias": 1, "gelu": 2, "residual": 3, "swiglu": 4, "bias_residual": 5, "relu": 6, "quick_gelu": 7}
+EPI = {None: 0, "bias": 1, "gelu": 2, "residual": 3, "swiglu": 4, "bias_residual": 5, "relu": 6, "quick_gelu": 7, "geglu": 10}
 _GEMM_KERNELS = {"auto": 0, "skinny": 1, "tiled": 2, "w4p": 8, "w4d": 9, "w4r": 10, "w4s": 11, "w4x": 12, "w4d192": 13,
                  # names of round-3 kernels that the persistent 256x256 kernels replaced
                  "large": 9, "ring": 10}
@@ -99,11 +99,12 @@ def linear(x: torch.Tensor, w: torch.Tensor, bias: Optional[torch.Tensor] = None
            out: Optional[torch.Tensor] = None) -> torch.Tensor:
     """y = act(x @ w^T + bias) + residual on the MFMA GEMM with a fused epilogue.
 
-    act: None | 'gelu' | 'relu' | 'quick_gelu' | 'swiglu' (w interleaved per 16 rows, see interleave_gate_up).
+    act: None | 'gelu' | 'relu' | 'quick_gelu' | 'swiglu' | 'geglu' (both with w interleaved per 16 rows, see
+    interleave_gate_up) | 'gelu_tanh'.
     An :class:`Fp8Weight` ``w`` routes to the fp8 MFMA GEMM (``linear_fp8``).
     """
-    if act in ("geglu", "gelu_tanh"):
-        # tanh-GELU family (Gemma GeGLU, StarCoder2 MLP): GEMM (+ bias) then one elementwise kernel
+    if act == "gelu_tanh" or (act == "geglu" and not _fused_glu_ok(x, w, bias)):
+        # tanh-GELU family (StarCoder2 MLP; GeGLU off the fused epilogue's grid): GEMM (+ bias) then one elementwise kernel
         assert residual is None and out is None
         y = linear(x, w, bias, out_dtype=None)
         y = geglu_interleaved(y) if act == "geglu" else gelu_tanh(y)
@@ -119,8 +120,8 @@ def linear(x: torch.Tensor, w: torch.Tensor, bias: Optional[torch.Tensor] = None
     lead = x.shape[:-1]
     M = x.numel() // K
     out_dtype = out_dtype or x.dtype
-    if act == "swiglu":
-        epi = EPI["swiglu"]
+    if act in ("swiglu", "geglu"):
+        epi = EPI[act]
         assert bias is None and residual is None
         ncol = N // 2
     elif act == "gelu":
@@ -150,6 +151,12 @@ def linear(x: torch.Tensor, w: torch.Tensor, bias: Optional[torch.Tensor] = None
         out = torch.empty(*lead, ncol, dtype=out_dtype, device=x.device)
     _native_gemm(x2, w, out, bias, residual, epi)
     return out
+
+
+def _fused_glu_ok(x, w, bias) -> bool:
+    """The GEMMs take the GeGLU epilogue: bf16 operands on their tile grid, no bias."""
+    return (x.is_cuda and isinstance(w, torch.Tensor) and bias is None and x.dtype == torch.bfloat16
+            and w.dtype == torch.bfloat16 and w.shape[1] % 64 == 0 and w.shape[0] % 32 == 0)
 
 
 def _vendor_linear(x, w, bias, residual, act, out_dtype, out):
@@ -870,6 +877,19 @@ def moe_route(logits: torch.Tensor, k: int, renorm: bool = True, score: str = "s
     w = torch.empty(T, k, dtype=torch.float32, device=logits.device)
     x = logits.float()
     native().moe_route(x if x.stride(1) == 1 else x.contiguous(), k, renorm, ids, w, score == "sigmoid", bias, float(eps))
+    return ids, w
+
+
+def moe_router(x: torch.Tensor, W: torch.Tensor, E: int, k: int, eps: float = 0.0):
+    """Router product, softmax scores over the E experts and the k largest -> (expert ids int32 [T, k], weights fp32 [T, k]
+    = chosen scores / (their sum + eps)). W [>= E, D] (rows past E: padding). One launch per decode-sized step, the router
+    GEMM and moe_route otherwise; logits are fp32 either way."""
+    T = x.shape[0]
+    if not x.is_cuda or T > 64:
+        return moe_route(linear(x, W, out_dtype=torch.float32)[:, :E], k, eps=eps)
+    ids = torch.empty(T, k, dtype=torch.int32, device=x.device)
+    w = torch.empty(T, k, dtype=torch.float32, device=x.device)
+    native().moe_router(x, W, E, k, float(eps), ids, w)
     return ids, w
 
 
