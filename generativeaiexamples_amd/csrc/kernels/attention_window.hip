@@ -887,7 +887,7 @@ void gai_rotary_half_kv_write(const void* q, int ldq, const void* k, int ldk, co
   const int wide = dt ? 4 : 8, per = DK / wide;   // 16-byte groups, one per lane when a head is a power of two of them
   const bool one = on_grid(wide) && per <= 64 && (per & (per - 1)) == 0;
   const bool two = on_grid(2);
-  const bool tiles = T >= 64;   // v in tiles of 16 tokens
+  const bool tiles = T >= 256;   // v in tiles of 16 tokens
   const int grid = T + (tiles ? (T + 15) / 16 : T);
 #define GAI_RH(TA, VEC_, NJ_, VT_)                                                                                   \
   rotary_half_kv_write_kernel<TA, VEC_, NJ_, VT_><<<grid, 256, lds, st>>>(                                           \

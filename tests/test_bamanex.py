@@ -199,7 +199,7 @@ def test_rotation_unit_norm_and_cache_write(device, dtype):
     g = torch.Generator().manual_seed(1)
     rn = lambda *s: torch.randn(*s, generator=g)  # noqa: E731
     dev = torch.device(device)
-    for T, H, G, dk, dv, rot in ((1, 2, 1, 64, 64, 32), (5, 3, 3, 7, 9, 4), (6, 4, 2, 128, 32, 128), (150, 5, 1, 48, 20, 16),
+    for T, H, G, dk, dv, rot in ((300, 4, 2, 64, 48, 32), (1, 2, 1, 64, 64, 32), (5, 3, 3, 7, 9, 4), (6, 4, 2, 128, 32, 128), (150, 5, 1, 48, 20, 16),
                                  (100, 2, 2, 16, 130, 16), (70, 1, 1, 256, 8, 64), (9, 2, 1, 200, 3, 0), (64, 6, 2, 8, 8, 6)):
         lens = (H * dk, G * dk, G * dv)
         x = rn(T, sum(lens) + 3).to(dtype)
@@ -215,7 +215,7 @@ def test_rotation_unit_norm_and_cache_write(device, dtype):
         inv = ops.rope_inv_freq(rot, 10000.0, rd["scaling"])
         assert torch.allclose(inv, torch.tensor(freqs, dtype=torch.float64), rtol=1e-12, atol=0)
         for eps in (None, 1e-5):
-            kc, vc = torch.zeros(20, G, B, dk, dtype=dtype, device=dev), torch.zeros(20, G, dv, B, dtype=dtype, device=dev)
+            kc, vc = torch.zeros(24, G, B, dk, dtype=dtype, device=dev), torch.zeros(24, G, dv, B, dtype=dtype, device=dev)
             xd = x.to(dev)
             q = ops.rotary_half_kv_write(*[xd[:, sum(lens[:i]):sum(lens[:i + 1])] for i in range(3)], pos.int().to(dev),
                                          slots.int().to(dev), kc, vc, H, G, dk, dv, inv.to(dev), eps)
