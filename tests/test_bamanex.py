@@ -129,7 +129,7 @@ MECHANISMS = {
     "experts-12-top5-tight": ([O.experts(O.att(), ff=40, n=12, top=5, limit=0.3, shared=8, shared_limit=0.2)], {}),
     "experts-all": ([O.experts(O.att(), n=4, top=4, limit=50.0)], {}),
     "experts-70": ([O.experts(O.att(), ff=4, n=70, top=16)], {}),
-    "loop-whole-stack": ([O.dense(O.att()), O.no_ff(O.att(window=4))], dict(loop=(0, 2, 3))),
+    "loop-whole-stack": ([O.dense(O.att()), O.no_ff(O.att(window=4))], dict(loop=(0, 2, 4))),
     "loop-once": ([O.dense(O.att()), O.no_ff(O.att(window=4))], dict(loop=(1, 2, 1))),
     "large-eps-unit-scale": ([O.dense(O.att(scale=1.0))], dict(eps=0.3, logit_scale=1.0)),
 }
